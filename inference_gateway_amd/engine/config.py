@@ -56,6 +56,11 @@ class RotarySpec:
     base: float = 10000.0
     dims: int = 0
 
+    def frequencies(self):
+        """([dims/2] angular steps as python floats, cos/sin factor)."""
+        return [self.base ** (-2.0 * i / self.dims)
+                for i in range(self.dims // 2)], 1.0
+
 
 @dataclass
 class MinGRUSpec:
@@ -72,7 +77,10 @@ class LatentAttentionSpec:
     q_rank: int = 64           # query latent width
     scale: float = 0.0         # score multiplier; 0 => (dim+rot_dim)**-0.5
     window: int = 0            # keys seen per query incl. itself; 0 = all
-    rot: RotarySpec = None
+    rot: object = None         # RotarySpec | YarnRotarySpec
+    rot_half: bool = False     # pairs (i, i + dims/2) instead of (2i, 2i+1)
+    sink: bool = True          # learned softmax sink per head
+    kv_from: int = -1          # layer whose cached rows are read (-1 = own)
 
     def __post_init__(self):
         if self.rot is None:
@@ -608,8 +616,8 @@ def feditar_preset(name: str, width: int, vocab: int, pattern: str,
 # ---------------------------------------------------------------------------
 @dataclass
 class YarnRotarySpec:
-    """Interleaved-pair rotary positions on the first `dims` entries of a
-    head with YaRN frequency interpolation: with where(t) = dims *
+    """Rotary positions on the first `dims` entries of a head (the pair
+    layout is the mixer's) with YaRN frequency interpolation: with where(t) = dims *
     ln(original / (2 pi t)) / (2 ln base), lo = max(floor(where(fast)),
     0), hi = min(ceil(where(slow)), dims - 1) and ramp_i = clamp((i - lo)
     / max(hi - lo, 0.001), 0, 1), pair i turns by position * (f_i /
@@ -644,6 +652,19 @@ class YarnRotarySpec:
             ramp = min(max((i - lo) / max(hi - lo, 0.001), 0.0), 1.0)
             out.append(fi / self.factor * ramp + fi * (1.0 - ramp))
         return out, 0.1 * math.log(self.factor) + 1.0
+
+    @staticmethod
+    def from_dict(r: Optional[dict]) -> "Optional[YarnRotarySpec]":
+        """A mixer's `rot` entry of config.json (None = no rotation)."""
+        if not r:
+            return None
+        sc = r.get("scaling") or {}
+        return YarnRotarySpec(
+            base=float(r["base"]), dims=int(r["dims"]),
+            factor=float(sc.get("factor") or 0.0),
+            original=float(sc.get("original") or 0.0),
+            fast=float(sc.get("fast", 32.0)),
+            slow=float(sc.get("slow", 1.0)))
 
 
 @dataclass
@@ -773,17 +794,6 @@ class BozolornConfig:
         """Parse the design's config.json (every size and constant is in
         it; `shapes` is accepted for symmetry with the other designs)."""
 
-        def rotary(r):
-            if not r:
-                return None
-            sc = r.get("scaling") or {}
-            return YarnRotarySpec(
-                base=float(r["base"]), dims=int(r["dims"]),
-                factor=float(sc.get("factor") or 0.0),
-                original=float(sc.get("original") or 0.0),
-                fast=float(sc.get("fast", 32.0)),
-                slow=float(sc.get("slow", 1.0)))
-
         def attention(m):
             kv_from = m.get("kv_from")
             return ChunkBiasAttentionSpec(
@@ -809,7 +819,7 @@ class BozolornConfig:
                         dim=int(a["dim"]),
                         vdim=int(a.get("vdim") or a["dim"]),
                         scale=float(a.get("scale") or 0.0),
-                        rot=rotary(a.get("rot"))),
+                        rot=YarnRotarySpec.from_dict(a.get("rot"))),
                     right=DeltaRuleSpec(
                         heads=int(b["heads"]),
                         kv_heads=int(b.get("kv_heads") or b["heads"]),
@@ -882,6 +892,181 @@ def bozolorn_preset(name: str, width: int, vocab: int, pattern: str,
     return BozolornConfig(name=name, hidden_size=width, vocab_size=vocab,
                           layers=layers, embed_scale=float(width) ** 0.5,
                           side_dim=side_dim)
+
+
+# ---------------------------------------------------------------------------
+# Bivatar: a per-layer post-norm decoder (the sublayers read the residual
+# itself; their RMS-normed outputs are added with one multiplier).  Mixers:
+# windowed softmax attention with the first tokens kept in sight, per-head
+# query/key norms and a linear distance bias, no rotation; or latent
+# attention with YaRN rotary positions on the shared key part, where a layer
+# may read another layer's cached latents.  Both gate every head's output
+# with one number.  Feed-forward: gelu-gated dense unit or none.
+# ---------------------------------------------------------------------------
+@dataclass
+class WindowAttentionSpec:
+    """Softmax attention with RMS-normed queries and keys (one weight
+    vector shared by the heads): score = q.k * scale - slope_h * (i - j),
+    slope_h = 2**(-8 (h + 1) / heads) (distance_bias off: no slope);
+    position i sees j <= i with i - j < window (0 = all) or j <
+    keep_first; one sigmoid output gate per head."""
+    heads: int = 1
+    kv_heads: int = 1
+    dim: int = 64
+    vdim: int = 64
+    scale: float = 0.0         # 0 => dim ** -0.5
+    window: int = 0
+    keep_first: int = 0
+    distance_bias: bool = True
+
+    def __post_init__(self):
+        if not self.scale:
+            self.scale = float(self.dim) ** -0.5
+        if self.heads % self.kv_heads:
+            raise ValueError("heads must be a multiple of kv_heads")
+
+
+@dataclass
+class GatedFFSpec:
+    """W_down (gelu_tanh(W_gate h) * (W_up h))."""
+    ff: int = 0
+
+
+@dataclass
+class BivatarConfig:
+    name: str
+    hidden_size: int
+    vocab_size: int
+    layers: list        # LayerSpec(type="attention"|"latent_attention")
+    norm_eps: float = 1e-6
+    embed_scale: float = 1.0
+    residual_mult: float = 1.0
+    max_position: int = 1 << 20     # angles are computed, not tabulated
+    architecture: str = "Bivatar"
+
+    def __post_init__(self):
+        for i, l in enumerate(self.layers):
+            if l.type != "latent_attention" or l.mixer.kv_from < 0:
+                continue
+            src = l.mixer.kv_from
+            if not (0 <= src < i) \
+                    or self.layers[src].type != "latent_attention" \
+                    or self.layers[src].mixer.kv_from >= 0:
+                raise ValueError(
+                    f"layer {i}: kv_from must name an earlier latent "
+                    "attention layer that projects its own keys")
+            o, m = self.layers[src].mixer, l.mixer
+            if (o.kv_rank, o.rot_dim, o.rot) != (m.kv_rank, m.rot_dim,
+                                                 m.rot):
+                raise ValueError(f"layer {i}: latent size or rotation "
+                                 f"differs from layer {src}'s")
+
+    @property
+    def num_layers(self) -> int:
+        return len(self.layers)
+
+    @property
+    def is_moe(self) -> bool:
+        return False
+
+    def kv_bytes_per_token(self, itemsize: int = 2) -> int:
+        """Paged bytes per token: keys and values of the windowed layers,
+        latent rows of the latent layers that own them."""
+        n = 0
+        for l in self.layers:
+            m = l.mixer
+            if l.type == "attention":
+                n += m.kv_heads * (m.dim + m.vdim) * itemsize
+            elif m.kv_from < 0:
+                n += m.cache_width * itemsize
+        return max(itemsize, n)
+
+    @staticmethod
+    def from_dict(cfg: dict, name: str = "bivatar",
+                  shapes: Optional[dict] = None) -> "BivatarConfig":
+        """Parse the design's config.json.  `shapes` (tensor name ->
+        shape, from the checkpoint header) fills sizes that the json
+        leaves to the tensors."""
+        shapes = shapes or {}
+        layers = []
+        for i, l in enumerate(cfg["layers"]):
+            m = l.get("mixer") or {}
+            t = l["type"]
+            if t == "attention":
+                mask = m.get("mask") or {}
+                mixer = WindowAttentionSpec(
+                    heads=int(m["heads"]),
+                    kv_heads=int(m.get("kv_heads") or m["heads"]),
+                    dim=int(m["dim"]), vdim=int(m.get("vdim") or m["dim"]),
+                    scale=float(m.get("scale") or 0.0),
+                    window=int(mask.get("size") or 0),
+                    keep_first=int(mask.get("keep_first") or 0))
+            elif t == "latent_attention":
+                kv_from = m.get("kv_from")
+                q_rank = m.get("q_rank")
+                if q_rank is None:
+                    q_rank = shapes[f"l{i}.mix.dq"][0]
+                rot = YarnRotarySpec.from_dict(m.get("rot"))
+                mixer = LatentAttentionSpec(
+                    heads=int(m["heads"]), dim=int(m["dim"]),
+                    rot_dim=int(m["rot_dim"]),
+                    vdim=int(m.get("vdim") or m["dim"]),
+                    kv_rank=int(m["kv_rank"]), q_rank=int(q_rank),
+                    scale=float(m.get("scale") or 0.0),
+                    window=int((m.get("mask") or {}).get("size") or 0),
+                    rot=rot, rot_half=True, sink=False,
+                    kv_from=-1 if kv_from is None else int(kv_from))
+            else:
+                raise ValueError(f"layer {i}: unknown mixer {t!r}")
+            f = l.get("mlp")
+            if f is None:
+                mlp = None
+            elif f["kind"] == "dense":
+                mlp = GatedFFSpec(ff=int(f["ff"]))
+            else:
+                raise ValueError(f"layer {i}: unknown mlp {f['kind']!r}")
+            layers.append(LayerSpec(type=t, mixer=mixer, mlp=mlp))
+        mult = cfg.get("residual_mult")
+        return BivatarConfig(
+            name=name, hidden_size=int(cfg["width"]),
+            vocab_size=int(cfg["vocab"]), layers=layers,
+            norm_eps=float((cfg.get("norm") or {}).get("eps", 1e-6)),
+            embed_scale=float((cfg.get("embedding") or {}).get("scale",
+                                                               1.0)),
+            residual_mult=1.0 if mult is None else float(mult))
+
+
+def bivatar_preset(name: str, width: int, vocab: int, pattern: str,
+                   heads: int, kv_heads: int, dim: int, vdim: int,
+                   window: int, keep_first: int, l_dim: int, rot_dim: int,
+                   l_vdim: int, kv_rank: int, q_rank: int, ff: int,
+                   rot_base: float = 10000.0, yarn_factor: float = 0.0,
+                   yarn_original: float = 0.0, residual_mult: float = 0.5,
+                   l_heads: int = 0) -> BivatarConfig:
+    """Layer pattern string: one token per layer — mixer `w` (windowed
+    attention), `l` (latent attention) or `l<j>` (the same, reading layer
+    j's latents), then `d` (dense) or `-` (no feed-forward); e.g. "wd ld
+    wd l1d"."""
+    layers = []
+    for tok in pattern.split():
+        if tok[0] == "w":
+            typ, mixer = "attention", WindowAttentionSpec(
+                heads=heads, kv_heads=kv_heads, dim=dim, vdim=vdim,
+                window=window, keep_first=keep_first)
+        else:
+            typ, mixer = "latent_attention", LatentAttentionSpec(
+                heads=l_heads or heads, dim=l_dim, rot_dim=rot_dim,
+                vdim=l_vdim, kv_rank=kv_rank, q_rank=q_rank,
+                rot=YarnRotarySpec(base=rot_base, dims=rot_dim,
+                                   factor=yarn_factor,
+                                   original=yarn_original),
+                rot_half=True, sink=False,
+                kv_from=int(tok[1:-1]) if tok[1:-1] else -1)
+        layers.append(LayerSpec(type=typ, mixer=mixer, mlp=GatedFFSpec(
+            ff=ff) if tok[-1] == "d" else None))
+    return BivatarConfig(name=name, hidden_size=width, vocab_size=vocab,
+                         layers=layers, embed_scale=float(width) ** 0.5,
+                         residual_mult=residual_mult)
 
 
 # Architectures from the public model cards (random-init weights — no network).
@@ -1057,6 +1242,19 @@ MODEL_PRESETS = {
         d_heads=32, d_kv_heads=8, d_dim=128, d_vdim=128, experts=8, top=2,
         groups=4, keep=2, expert_ff=14336, side_dim=64,
         yarn_factor=4.0, yarn_original=4096.0),
+    # tiny Bivatar for CPU tests / smoke: both mixers, a layer that reads
+    # another's latents, a layer without feed-forward
+    "tiny-bivatar": bivatar_preset(
+        "tiny-bivatar", width=96, vocab=320, pattern="wd ld w- l1d",
+        heads=4, kv_heads=2, dim=24, vdim=16, window=20, keep_first=3,
+        l_dim=16, rot_dim=8, l_vdim=24, kv_rank=40, q_rank=48, ff=160,
+        yarn_factor=4.0, yarn_original=64.0),
+    # layer-shape benchmark point at Llama-3-8B's width
+    "bivatar-4k": bivatar_preset(
+        "bivatar-4k", width=4096, vocab=32000, pattern="wd ld wd l1d",
+        heads=32, kv_heads=8, dim=128, vdim=128, window=1024,
+        keep_first=16, l_dim=128, rot_dim=64, l_vdim=128, kv_rank=512,
+        q_rank=1536, ff=14336, yarn_factor=8.0, yarn_original=4096.0),
     "tiny-moe": ModelConfig(
         name="tiny-moe",
         hidden_size=512,
@@ -1210,6 +1408,19 @@ class EngineConfig:
     def tiny_bozolorn(**kw) -> "EngineConfig":
         defaults = dict(
             model=MODEL_PRESETS["tiny-bozolorn"],
+            num_gpu_blocks=64,
+            max_num_seqs=8,
+            max_batched_tokens=2048,
+            max_model_len=512,
+            use_hip_graphs=False,
+        )
+        defaults.update(kw)
+        return EngineConfig(**defaults)
+
+    @staticmethod
+    def tiny_bivatar(**kw) -> "EngineConfig":
+        defaults = dict(
+            model=MODEL_PRESETS["tiny-bivatar"],
             num_gpu_blocks=64,
             max_num_seqs=8,
             max_batched_tokens=2048,

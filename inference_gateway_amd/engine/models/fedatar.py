@@ -97,7 +97,10 @@ class LatentAttention(nn.Module):
     (q_abs = W_uk^T q_unrotated) and the value up-projection is applied
     after the probability-weighted sum of latents, so every head reads
     the same cached row (latent | rotated key) — prefill portions and
-    decoded tokens both attend straight out of the paged cache."""
+    decoded tokens both attend straight out of the paged cache.  The
+    per-head output gate is applied to the latent sum (it commutes with
+    the value up-projection).  A layer with spec.kv_from >= 0 has no
+    key/value projection and reads the rows of that layer."""
 
     cache_kind = "latent"
 
@@ -109,14 +112,17 @@ class LatentAttention(nn.Module):
         H, dn, rd = spec.heads, spec.dim, spec.rot_dim
         R, vd, qr = spec.kv_rank, spec.vdim, spec.q_rank
         s = hidden ** -0.5 / 0.02
+        self.owns_kv = spec.kv_from < 0
         # fused down projection: query latent | kv latent | rotated key
-        # | per-head output-gate logits
-        self.down = _param(_rand((qr + R + rd + H, hidden), device, dtype,
+        # (own keys only) | per-head output-gate logits
+        rows = qr + (R + rd if self.owns_kv else 0) + H
+        self.down = _param(_rand((rows, hidden), device, dtype,
                                  name + ".down", s))
         self.qnorm_w = _param(1.0 + _rand((qr,), device, torch.float32,
                                           name + ".qn", 2.0))
-        self.kvnorm_w = _param(1.0 + _rand((R,), device, torch.float32,
-                                           name + ".kvn", 2.0))
+        self.kvnorm_w = _param(1.0 + _rand(
+            (R,), device, torch.float32, name + ".kvn", 2.0)) \
+            if self.owns_kv else None
         self.uq = _param(_rand((H * (dn + rd), qr), device, dtype,
                                name + ".uq", qr ** -0.5 / 0.02))
         # absorbed forms, per head: uk [H, dn, R] maps an unrotated query
@@ -126,34 +132,45 @@ class LatentAttention(nn.Module):
         self.uv_t = _param(_rand((H, R, vd), device, dtype, name + ".uv",
                                  R ** -0.5 / 0.02))
         self.sink = _param(_rand((H,), device, torch.float32,
-                                 name + ".sink", 25.0))
+                                 name + ".sink", 25.0)) \
+            if spec.sink else None
         self.o = _param(_rand((hidden, H * vd), device, dtype, name + ".o",
                               (H * vd) ** -0.5 / 0.02))
-        self.inv_freq = _param(ops.rotary_inv_freq(
-            spec.rot.base, spec.rot.dims, device))
+        freq, self.mag = spec.rot.frequencies()
+        self.inv_freq = _param(torch.tensor(
+            freq, dtype=torch.float64).to(torch.float32).to(device))
 
     def cache_width(self) -> int:
         return self.spec.cache_width
 
+    def cache_spec(self) -> tuple:
+        return ("latent", self.cache_width()) if self.owns_kv \
+            else ("group", [])
+
     def forward(self, h: torch.Tensor, fb: ForwardBatch,
                 cache: torch.Tensor) -> torch.Tensor:
+        """cache: this layer's paged rows, or its source layer's."""
         sp = self.spec
         T = h.shape[0]
         H, dn, rd = sp.heads, sp.dim, sp.rot_dim
         down = F.linear(h, self.down)
         cq, gate = ops.latent_down_post(
-            down, fb.positions, fb.slot_mapping, cache, self.qnorm_w,
-            self.kvnorm_w, self.inv_freq, self.eps, sp.q_rank, sp.kv_rank,
-            rd, H)
+            down, fb.positions, fb.slot_mapping,
+            cache if self.owns_kv else None, self.qnorm_w, self.kvnorm_w,
+            self.inv_freq, self.eps, sp.q_rank, sp.kv_rank, rd, H,
+            sp.rot_half, self.mag)
         q = F.linear(cq, self.uq).view(T, H, dn + rd)
-        ops.rope_pairs_(q, fb.positions, self.inv_freq, dn)
+        ops.rope_pairs_(q, fb.positions, self.inv_freq, dn, sp.rot_half,
+                        self.mag)
         q_abs = torch.bmm(q[:, :, :dn].transpose(0, 1), self.uk)  # [H,T,R]
         o_lat = ops.latent_attention(
             q_abs.transpose(0, 1), q[:, :, dn:], cache, fb.seq_block_table,
             fb.row_seq, fb.positions, self.sink, sp.scale, sp.window,
-            fb.num_chunk_rows, fb.seq_lens, fb.max_context)
-        v = torch.bmm(o_lat.transpose(0, 1), self.uv_t)           # [H,T,vd]
-        return F.linear(ops.gate_heads(v, gate), self.o)
+            fb.num_chunk_rows, fb.seq_lens, fb.max_context, gate)
+        # the batched product writes head-major rows [T, H, vd] in place
+        v = torch.empty((T, H, sp.vdim), dtype=h.dtype, device=h.device)
+        torch.bmm(o_lat.transpose(0, 1), self.uv_t, out=v.transpose(0, 1))
+        return F.linear(v.view(T, H * sp.vdim), self.o)
 
 
 class XieluMLP(nn.Module):

@@ -8,8 +8,8 @@ from pathlib import Path
 
 import torch
 
-from ..config import (BozolornConfig, FedatarConfig, FeditarConfig,
-                      MekevikConfig, ModelConfig)
+from ..config import (BivatarConfig, BozolornConfig, FedatarConfig,
+                      FeditarConfig, MekevikConfig, ModelConfig)
 
 
 def build_model(model_cfg, device, dtype):
@@ -22,6 +22,8 @@ def build_model(model_cfg, device, dtype):
         from .feditar import FeditarForCausalLM as cls
     elif isinstance(model_cfg, BozolornConfig):
         from .bozolorn import BozolornForCausalLM as cls
+    elif isinstance(model_cfg, BivatarConfig):
+        from .bivatar import BivatarForCausalLM as cls
     elif model_cfg.is_moe:
         from .mixtral import MixtralForCausalLM as cls
     else:
@@ -66,6 +68,10 @@ def model_config_from_dir(path: str):
         return BozolornConfig.from_dict(
             cfg, name=Path(path).name or "bozolorn",
             shapes=safetensors_shapes(path))
+    if cfg.get("architecture") == "Bivatar":
+        return BivatarConfig.from_dict(
+            cfg, name=Path(path).name or "bivatar",
+            shapes=safetensors_shapes(path))
     if cfg.get("architecture") == "Fedatar":
         return FedatarConfig.from_dict(
             cfg, name=Path(path).name or "fedatar",
@@ -90,4 +96,4 @@ def is_recurrent(model_cfg) -> bool:
 
 __all__ = ["build_model", "model_config_from_dir", "safetensors_shapes",
            "is_recurrent", "ModelConfig", "FedatarConfig", "MekevikConfig",
-           "FeditarConfig", "BozolornConfig"]
+           "FeditarConfig", "BozolornConfig", "BivatarConfig"]

@@ -561,6 +561,58 @@ def load_bozolorn_weights(model, path: str) -> int:
     return n
 
 
+def load_bivatar_weights(model, path: str) -> int:
+    """Load a Bivatar checkpoint: tensors `embed`, `l<i>.norm1|norm2`,
+    `l<i>.mix.*` per mixer kind, `l<i>.mlp.{gate,up,down}`, `final.norm`,
+    `head`.  The engine's layouts are assembled here: q|k|v|g stacked for
+    the windowed attention's input GEMM; dq|dkv|g (dq|g for a layer that
+    reads another layer's latents) for the latent attention's, whose key
+    and value up-projections are kept per head in absorbed form; gate|up
+    stacked for the feed-forward.  Norm weights are held in fp32."""
+    sh = _Shards(path)
+    cfg = model.cfg
+    n = 0
+
+    def put(param, src, what):
+        nonlocal n
+        _copy(param, src, what)
+        n += 1
+
+    def cat(prefix, names):
+        return torch.cat([sh.full(prefix + c) for c in names], 0)
+
+    put(model.embed, sh.full("embed"), "embed")
+    for i, (spec, layer) in enumerate(zip(cfg.layers, model.layers)):
+        p = f"l{i}."
+        put(layer.norm1_w, sh.full(p + "norm1"), p + "norm1")
+        mx, m, a = layer.mixer, p + "mix.", spec.mixer
+        if spec.type == "attention":
+            put(mx.qkvg, cat(m, "qkvg"), m + "q|k|v|g")
+            put(mx.qnorm_w, sh.full(m + "q.norm"), m + "q.norm")
+            put(mx.knorm_w, sh.full(m + "k.norm"), m + "k.norm")
+        else:
+            rows = ("dq", "dkv", "g") if mx.owns_kv else ("dq", "g")
+            put(mx.down, cat(m, rows), m + "|".join(rows))
+            put(mx.qnorm_w, sh.full(m + "dq.norm"), m + "dq.norm")
+            if mx.owns_kv:
+                put(mx.kvnorm_w, sh.full(m + "dkv.norm"), m + "dkv.norm")
+            put(mx.uq, sh.full(m + "uq"), m + "uq")
+            put(mx.uk, sh.full(m + "uk").view(a.heads, a.dim, a.kv_rank),
+                m + "uk")
+            put(mx.uv_t, sh.full(m + "uv").view(
+                a.heads, a.vdim, a.kv_rank).transpose(1, 2), m + "uv")
+        put(mx.o, sh.full(m + "o"), m + "o")
+        if spec.mlp is None:
+            continue
+        put(layer.norm2_w, sh.full(p + "norm2"), p + "norm2")
+        put(layer.mlp.gate_up, cat(p + "mlp.", ("gate", "up")),
+            p + "mlp.gate|up")
+        put(layer.mlp.down, sh.full(p + "mlp.down"), p + "mlp.down")
+    put(model.final_norm_w, sh.full("final.norm"), "final.norm")
+    put(model.head, sh.full("head"), "head")
+    return n
+
+
 def _is_gguf(path: str) -> bool:
     p = Path(path)
     if p.is_file():
@@ -588,6 +640,8 @@ def load_weights(model, path: str) -> int:
         return load_feditar_weights(model, path)
     if getattr(model.cfg, "architecture", "") == "Bozolorn":
         return load_bozolorn_weights(model, path)
+    if getattr(model.cfg, "architecture", "") == "Bivatar":
+        return load_bivatar_weights(model, path)
     if getattr(model.cfg, "is_moe", False):
         return load_mixtral_weights(model, path)
     return load_llama_weights(model, path)

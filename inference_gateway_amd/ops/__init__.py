@@ -40,6 +40,15 @@ except ImportError:  # pragma: no cover - absent only before first build
     HAS_RECURRENT = False
 
 
+try:
+    from . import _postnorm  # windowed + latent attention, post-norm steps
+
+    HAS_POSTNORM = True
+except ImportError:  # pragma: no cover - absent only before first build
+    _postnorm = None
+    HAS_POSTNORM = False
+
+
 def _require_recurrent() -> None:
     if not HAS_RECURRENT:
         raise RuntimeError(
@@ -51,13 +60,16 @@ def _require_recurrent() -> None:
 
 
 def _shared_ext(name: str):
-    """The row-wise ops that both the hybrid and the recurrent extension
-    compile (same source file): whichever is loaded serves them, so a
-    process that runs one model family loads one library."""
-    for ext in (_hybrid, _recurrent):
+    """An op that several extensions compile (same source file):
+    whichever is built serves it, so a process that runs one model family
+    needs one library."""
+    for ext in (_postnorm, _hybrid, _recurrent):
         if ext is not None and hasattr(ext, name):
             return getattr(ext, name)
-    _require_hybrid()
+    raise RuntimeError(
+        f"no built kernel extension has {name!r} but a GPU tensor was "
+        "passed. Build them in-tree with: PYTORCH_ROCM_ARCH=gfx950 python "
+        "setup.py build_ext --inplace")
 
 
 def _require_hybrid() -> None:
@@ -328,36 +340,42 @@ def mingru_scan(zug, state, seq_cu, seq_start, seq_slots, seq_rows):
                                      seq_slots)
 
 
-def rope_pairs_(x, positions, inv_freq, offset: int):
-    """In-place interleaved-pair rotation of x[T, H, hd][..., offset :
-    offset + 2*len(inv_freq)] by positions * inv_freq (fp32 angles)."""
+def rope_pairs_(x, positions, inv_freq, offset: int, half: bool = False,
+                mag: float = 1.0):
+    """In-place rotation of x[T, H, hd][..., offset : offset +
+    2*len(inv_freq)] by positions * inv_freq (fp32 angles), cos and sin
+    times `mag`.  Pairs are (2i, 2i+1), or with `half` (i, i +
+    len(inv_freq))."""
     if x.is_cuda:
-        _require_hybrid()
-        _hybrid.rope_pairs(x, positions, inv_freq, offset)
+        _shared_ext("rope_pairs")(x, positions, inv_freq, offset, half, mag)
         return x
-    return torch_ref.rope_pairs_ref(x, positions, inv_freq, offset)
+    return torch_ref.rope_pairs_ref(x, positions, inv_freq, offset, half,
+                                    mag)
 
 
 def latent_down_post(down, positions, slot_mapping, cache, qnorm_w,
                      kvnorm_w, inv_freq, eps: float, q_rank: int,
-                     kv_rank: int, rot_dim: int, heads: int):
+                     kv_rank: int, rot_dim: int, heads: int,
+                     half: bool = False, mag: float = 1.0):
     """Post-processing of the fused down projection [T, q_rank + kv_rank
     + rot_dim + heads]: returns (normed query latent [T, q_rank],
     sigmoid head gates [T, heads] fp32) and appends (normed latent |
-    rotated shared key) to the paged cache at slot_mapping."""
+    rotated shared key) to the paged cache at slot_mapping; half and mag
+    as in rope_pairs_.  cache None: the layer reads another layer's rows,
+    down is [T, q_rank + heads] and nothing is appended."""
     if down.is_cuda:
-        _require_hybrid()
         T = down.shape[0]
         cq = torch.empty((T, q_rank), dtype=down.dtype, device=down.device)
         gate = torch.empty((T, heads), dtype=torch.float32,
                            device=down.device)
-        _hybrid.latent_down_post(cq, gate, down, positions, slot_mapping,
-                                  cache, qnorm_w, kvnorm_w, inv_freq, eps,
-                                  q_rank, kv_rank, rot_dim, heads)
+        _shared_ext("latent_down_post")(
+            cq, gate, down, positions, slot_mapping, cache, qnorm_w,
+            kvnorm_w, inv_freq, eps, q_rank, kv_rank, rot_dim, heads, half,
+            mag)
         return cq, gate
     return torch_ref.latent_down_post_ref(
         down, positions, slot_mapping, cache, qnorm_w, kvnorm_w, inv_freq,
-        eps, q_rank, kv_rank, rot_dim, heads)
+        eps, q_rank, kv_rank, rot_dim, heads, half, mag)
 
 
 import functools
@@ -404,9 +422,11 @@ LATENT_ATTENTION_MFMA = True
 def latent_attention(q_abs, q_rot, cache, block_table, row_seq, positions,
                      sink, scale: float, window: int,
                      num_prefill_rows: int = 0, prefill_seq_lens=None,
-                     max_context: int = 0):
+                     max_context: int = 0, gate=None):
     """Absorbed latent attention (all heads share one cached latent per
-    token) with a sliding window and a per-head softmax sink.
+    token) with a sliding window (0 = causal), a per-head softmax sink
+    (None = ordinary softmax) and an output gate per head (gate [T, H]
+    fp32, None = 1).
     q_abs [T, H, kv_rank], q_rot [T, H, rot_dim] (strided views ok),
     cache [blocks, block, kv_rank + rot_dim].  Rows [0, num_prefill_rows)
     are prompt portions (prefill_seq_lens = python row counts per
@@ -414,27 +434,28 @@ def latent_attention(q_abs, q_rot, cache, block_table, row_seq, positions,
     hint (longest sequence in the batch) for splitting keys over
     workgroups."""
     if q_abs.is_cuda:
-        _require_hybrid()
         T, H, R = q_abs.shape
         out = torch.empty((T, H, R), dtype=q_abs.dtype, device=q_abs.device)
         if q_abs.dtype == torch.bfloat16 and LATENT_ATTENTION_MFMA:
             tiles = _attention_tiles(
-                _hybrid.latent_attention_tile_rows(H), num_prefill_rows,
+                _shared_ext("latent_attention_tile_rows")(H),
+                num_prefill_rows,
                 tuple(prefill_seq_lens or ()) if num_prefill_rows else (),
                 T, q_abs.device)
             ctx = max_context or 4096
             max_keys = min(window, ctx) if window > 0 else ctx
-            if _hybrid.latent_attention_mfma(
+            if _shared_ext("latent_attention_mfma")(
                     out, q_abs, q_rot, cache, block_table, row_seq,
                     positions, tiles[0], tiles[1], sink, scale, window,
-                    max_keys):
+                    max_keys, gate):
                 return out
-        _hybrid.latent_attention(out, q_abs, q_rot, cache, block_table,
-                                 row_seq, positions, sink, scale, window)
+        _shared_ext("latent_attention")(
+            out, q_abs, q_rot, cache, block_table, row_seq, positions, sink,
+            scale, window, gate)
         return out
     return torch_ref.latent_attention_ref(
         q_abs, q_rot, cache, block_table, row_seq, positions, sink, scale,
-        window)
+        window, gate)
 
 
 def xielu(z, pq):
@@ -498,6 +519,7 @@ def moe_topk_route(logits, top_k: int, capacity: int = 0,
 # ---------------------------------------------------------------------------
 GATED_ACT_SILU = torch_ref.GATED_ACT_SILU
 GATED_ACT_CLAMPED = torch_ref.GATED_ACT_CLAMPED
+GATED_ACT_GELU = torch_ref.GATED_ACT_GELU
 
 
 def add_rmsnorm_pair(residual, delta_a, delta_b, w1, w2, eps: float,
@@ -588,7 +610,8 @@ def sigmoid_attention(q, kcache, vcache, block_table, row_seq, positions,
 def gated_act(gate_up, mode: int, limit: float = 0.0, alpha: float = 1.0):
     """(gate | up) halves of the last dim -> one activation:
     GATED_ACT_SILU silu(g) * u; GATED_ACT_CLAMPED with g' = min(g, limit),
-    u' = clamp(u, -limit, limit): g' * sigmoid(alpha g') * (u' + 1)."""
+    u' = clamp(u, -limit, limit): g' * sigmoid(alpha g') * (u' + 1);
+    GATED_ACT_GELU gelu_tanh(g) * u."""
     if gate_up.is_cuda:
         f = gate_up.shape[-1] // 2
         out = torch.empty((*gate_up.shape[:-1], f), dtype=gate_up.dtype,
@@ -765,7 +788,7 @@ def _softcap_tiles(seq_lens: tuple, num_seqs: int, device):
     len(seq_lens) sequences of the batch) cut into runs of its tile rows,
     and the sequences that bring one decoded row.  Cached: serving
     repeats the same batch shapes."""
-    tq = int(_recurrent.softcap_attention_tile_rows())
+    tq = int(_shared_ext("softcap_attention_tile_rows")())
     tseq, toff = torch_ref.make_prefill_tiles(seq_lens, tq, device)
     dec = torch.arange(len(seq_lens), num_seqs, dtype=torch.int32,
                        device=device)
@@ -777,23 +800,25 @@ def softcap_attention(q, kcache, vcache, block_table, row_seq, positions,
                       temp_coef: float = 0.0, temp_every: int = 1,
                       window: int = 0, num_prefill_rows: int = 0,
                       prefill_seq_lens=None, seq_cu=None, seq_start=None,
-                      slopes=None, chunk: int = 0, sinks=None, gate=None):
+                      slopes=None, chunk: int = 0, sinks=None, gate=None,
+                      keep: int = 0):
     """Causal softmax attention over paged keys/values with grouped
     heads and separate key and value widths.  score = (q . k) * scale *
     (1 + temp_coef * ln(floor((p + 1) / temp_every) + 1)), squashed by
     softcap * tanh(. / softcap) when softcap > 0; window > 0 keeps the
-    last `window` keys.  Optional: slopes [H] fp32 take slope_h * (p - j)
+    last `window` keys, and keep > 0 the first `keep` keys of the
+    sequence whatever window and chunk say.  Optional: slopes [H] fp32 take slope_h * (p - j)
     off the score of key j; chunk > 0 keeps only the keys from floor(p /
     chunk) * chunk on; sinks [H] fp32 add exp(sink_h) to the softmax
-    denominator (a key with that score and no value); gate [T, H*P]
-    (strided rows ok) multiplies the result by sigmoid(gate).
+    denominator (a key with that score and no value); gate [T, H*P] or
+    [T, H] (strided rows ok) multiplies the result by sigmoid(gate), per
+    value entry or per head.
     q [T, H*N] (strided ok) -> [T, H*P].  Rows [0,
     num_prefill_rows) are prompt portions (prefill_seq_lens = python row
     counts of the first sequences), the rest single decoded tokens;
     seq_cu / seq_start describe the sequences (needed by the tile
     kernel; without them every batch runs the row kernel)."""
     if q.is_cuda:
-        _require_recurrent()
         T = q.shape[0]
         H = q.shape[1] // kcache.shape[3]
         out = torch.empty((T, H * vcache.shape[3]), dtype=q.dtype,
@@ -803,19 +828,19 @@ def softcap_attention(q, kcache, vcache, block_table, row_seq, positions,
             lens = tuple(prefill_seq_lens or ()) if num_prefill_rows else ()
             tseq, toff, dec = _softcap_tiles(lens, seq_start.shape[0],
                                              q.device)
-            if _recurrent.softcap_attention_mfma(
+            if _shared_ext("softcap_attention_mfma")(
                     out, q, kcache, vcache, block_table, seq_cu, seq_start,
                     tseq, toff, dec, scale, softcap, temp_coef, temp_every,
-                    window, slopes, chunk, sinks, gate):
+                    window, slopes, chunk, sinks, gate, keep):
                 return out
-        _recurrent.softcap_attention(out, q, kcache, vcache, block_table,
-                                     row_seq, positions, scale, softcap,
-                                     temp_coef, temp_every, window, slopes,
-                                     chunk, sinks, gate)
+        _shared_ext("softcap_attention")(
+            out, q, kcache, vcache, block_table, row_seq, positions, scale,
+            softcap, temp_coef, temp_every, window, slopes, chunk, sinks,
+            gate, keep)
         return out
     return recurrent_ref.softcap_attention_ref(
         q, kcache, vcache, block_table, row_seq, positions, scale, softcap,
-        temp_coef, temp_every, window, slopes, chunk, sinks, gate)
+        temp_coef, temp_every, window, slopes, chunk, sinks, gate, keep)
 
 
 def qk_norm_rope_append(proj, positions, slot_mapping, kcache, vcache,
@@ -830,13 +855,11 @@ def qk_norm_rope_append(proj, positions, slot_mapping, kcache, vcache,
     appended to the paged caches [blocks, kv_heads, block, dim | vdim].
     Returns the queries [T, heads*dim]."""
     if proj.is_cuda:
-        _require_recurrent()
         q = torch.empty((proj.shape[0], heads * dim), dtype=proj.dtype,
                         device=proj.device)
-        _recurrent.qk_norm_rope_append(q, proj, positions, slot_mapping,
-                                       kcache, vcache, qnorm_w, knorm_w,
-                                       inv_freq, mag, eps, heads, kv_heads,
-                                       dim, vdim)
+        _shared_ext("qk_norm_rope_append")(
+            q, proj, positions, slot_mapping, kcache, vcache, qnorm_w,
+            knorm_w, inv_freq, mag, eps, heads, kv_heads, dim, vdim)
         return q
     return recurrent_ref.qk_norm_rope_append_ref(
         proj, positions, slot_mapping, kcache, vcache, qnorm_w, knorm_w,
@@ -911,20 +934,19 @@ def moe_group_route(logits, correction, top_k: int, groups: int, keep: int,
 
 
 def add_normed_rmsnorm(residual, delta, w_post, w_pre, eps: float,
-                       out_dtype):
-    """Sandwich-norm step: residual [T, D] fp32 += rmsnorm(delta) *
-    w_post (in place; delta None = nothing added), then returns
-    rmsnorm(residual) * w_pre in out_dtype (w_pre None: the residual
-    itself in out_dtype).  Weights fp32 [D]."""
+                       out_dtype, mult: float = 1.0):
+    """Step of a layer that norms its sublayers' outputs: residual [T, D]
+    fp32 += mult * rmsnorm(delta) * w_post (in place; delta None = nothing
+    added), then returns rmsnorm(residual) * w_pre in out_dtype (w_pre
+    None: the residual itself in out_dtype).  Weights fp32 [D]."""
     if residual.is_cuda:
-        _require_recurrent()
         out = torch.empty(residual.shape, dtype=out_dtype,
                           device=residual.device)
-        _recurrent.add_normed_rmsnorm(out, residual, delta, w_post, w_pre,
-                                      eps)
+        _shared_ext("add_normed_rmsnorm")(out, residual, delta, w_post,
+                                          w_pre, eps, mult)
         return out
     return recurrent_ref.add_normed_rmsnorm_ref(residual, delta, w_post,
-                                                w_pre, eps, out_dtype)
+                                                w_pre, eps, out_dtype, mult)
 
 
 def gelu_mul_rows(z, table, tokens, col0: int):

@@ -44,6 +44,19 @@ DEVINLINE float sigmoid_for<float>(float x) { return sigmoid_f32(x); }
 template <>
 DEVINLINE float sigmoid_for<uint16_t>(float x) { return sigmoid_fast(x); }
 
+// optional per-head fp32 vectors of an attention launch: sinks [H] and
+// output gates [T, H]
+static inline void check_head_vectors(
+    const c10::optional<torch::Tensor>& sink,
+    const c10::optional<torch::Tensor>& gate, int64_t T, int64_t H) {
+  if (sink.has_value())
+    TORCH_CHECK(sink->dtype() == torch::kFloat32 && sink->is_contiguous() &&
+                sink->numel() == H);
+  if (gate.has_value())
+    TORCH_CHECK(gate->dtype() == torch::kFloat32 && gate->is_contiguous() &&
+                gate->numel() == T * H);
+}
+
 #define IGW_DISPATCH_ACT(TENSOR, ...)                                   \
   do {                                                                  \
     if ((TENSOR).scalar_type() == torch::kBFloat16) {                   \

@@ -10,12 +10,15 @@ void add_layernorm(torch::Tensor out, torch::Tensor residual,
                    torch::Tensor bias, double eps);
 void latent_down_post(torch::Tensor cq, torch::Tensor gate, torch::Tensor down,
                       torch::Tensor positions, torch::Tensor slot_mapping,
-                      torch::Tensor cache, torch::Tensor qnorm_w,
-                      torch::Tensor kvnorm_w, torch::Tensor inv_freq,
-                      double eps, int64_t q_rank, int64_t kv_rank,
-                      int64_t rot_dim, int64_t heads);
+                      c10::optional<torch::Tensor> cache,
+                      torch::Tensor qnorm_w,
+                      c10::optional<torch::Tensor> kvnorm_w,
+                      torch::Tensor inv_freq, double eps, int64_t q_rank,
+                      int64_t kv_rank, int64_t rot_dim, int64_t heads,
+                      bool half, double mag);
 void rope_pairs(torch::Tensor x, torch::Tensor positions,
-                torch::Tensor inv_freq, int64_t offset);
+                torch::Tensor inv_freq, int64_t offset, bool half,
+                double mag);
 void xielu(torch::Tensor out, torch::Tensor in, torch::Tensor pq);
 void relu2(torch::Tensor out, torch::Tensor in);
 void gate_heads(torch::Tensor out, torch::Tensor v, torch::Tensor gate);
@@ -54,14 +57,17 @@ void mingru_scan_chunked(torch::Tensor y, torch::Tensor zug,
 void latent_attention(torch::Tensor out, torch::Tensor q_abs,
                       torch::Tensor q_rot, torch::Tensor cache,
                       torch::Tensor block_table, torch::Tensor row_seq,
-                      torch::Tensor positions, torch::Tensor sink,
-                      double scale, int64_t window);
+                      torch::Tensor positions,
+                      c10::optional<torch::Tensor> sink, double scale,
+                      int64_t window, c10::optional<torch::Tensor> gate);
 bool latent_attention_mfma(torch::Tensor out, torch::Tensor q_abs,
                            torch::Tensor q_rot, torch::Tensor cache,
                            torch::Tensor block_table, torch::Tensor row_seq,
                            torch::Tensor positions, torch::Tensor tile_row0,
-                           torch::Tensor tile_nrows, torch::Tensor sink,
-                           double scale, int64_t window, int64_t max_keys);
+                           torch::Tensor tile_nrows,
+                           c10::optional<torch::Tensor> sink, double scale,
+                           int64_t window, int64_t max_keys,
+                           c10::optional<torch::Tensor> gate);
 int64_t latent_attention_tile_rows(int64_t H);
 bool sigmoid_attention_mfma(torch::Tensor out, torch::Tensor q,
                             torch::Tensor kcache, torch::Tensor vcache,
@@ -80,7 +86,7 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("latent_down_post", &igw::latent_down_post,
         "latent RMS norms + shared-key rotation + paged append + head gates");
   m.def("rope_pairs", &igw::rope_pairs,
-        "in-place interleaved-pair rotary on a slice of every head");
+        "in-place rotary on a slice of every head, interleaved or half pairs");
   m.def("xielu", &igw::xielu, "xIELU activation");
   m.def("relu2", &igw::relu2, "squared ReLU activation");
   m.def("gate_heads", &igw::gate_heads,
@@ -92,7 +98,7 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("qk_norm_append", &igw::qk_norm_append,
         "whole-projection query/key RMS norms + value blend + paged append");
   m.def("gated_act", &igw::gated_act,
-        "(gate | up) -> silu(g) u or the clamped gated unit");
+        "(gate | up) -> silu(g) u, the clamped gated unit or gelu_tanh(g) u");
   m.def("sigmoid_attention", &igw::sigmoid_attention,
         "windowed sigmoid attention, distance bias, head mixing, paged");
   m.def("sigmoid_attention_mfma", &igw::sigmoid_attention_mfma,
@@ -105,7 +111,7 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("mingru_scan_chunked", &igw::mingru_scan_chunked,
         "minGRU recurrence as a three-pass chunked scan");
   m.def("latent_attention", &igw::latent_attention,
-        "absorbed latent attention, sliding window + softmax sink, paged");
+        "absorbed latent attention, window, softmax sink, head gate, paged");
   m.def("latent_attention_mfma", &igw::latent_attention_mfma,
         "absorbed latent attention on MFMA tiles (bf16); false = sizes do "
         "not fit, use latent_attention");

@@ -93,14 +93,24 @@ void add_layernorm(torch::Tensor out, torch::Tensor residual,
 }
 
 // ---------------------------------------------------------------------------
+// Rotary pairs of n_pairs angles: interleaved (2i, 2i+1) or, HALF, entry i
+// with entry i + n_pairs.  cos and sin are multiplied by `mag`.
+DEVINLINE void rotary_pair_index(bool half, int i, int n_pairs, int& a,
+                                 int& b) {
+  a = half ? i : 2 * i;
+  b = half ? i + n_pairs : 2 * i + 1;
+}
+
+// cache == nullptr: the layer owns no keys, down holds q_rank | heads only
+// (R = RD = n_pairs = 0)
 template <typename T>
 __global__ __launch_bounds__(ROW_BLOCK) void latent_down_post_kernel(
     T* __restrict__ cq, float* __restrict__ gate, const T* __restrict__ down,
     int64_t down_stride, const int32_t* __restrict__ positions,
     const int32_t* __restrict__ slot_mapping, T* __restrict__ cache,
     const float* __restrict__ wq, const float* __restrict__ wc,
-    const float* __restrict__ inv_freq, int n_pairs, float eps, int QR, int R,
-    int RD, int H) {
+    const float* __restrict__ inv_freq, int n_pairs, bool half, float mag,
+    float eps, int QR, int R, int RD, int H) {
   __shared__ float lds_a[ROW_BLOCK / 64], lds_b[ROW_BLOCK / 64];
   const int64_t t = blockIdx.x;
   const T* x = down + t * down_stride;
@@ -114,39 +124,52 @@ __global__ __launch_bounds__(ROW_BLOCK) void latent_down_post_kernel(
     sc += v * v;
   }
   const float rq = 1.0f / sqrtf(row_block_sum(sq, lds_a) / (float)QR + eps);
-  const float rc = 1.0f / sqrtf(row_block_sum(sc, lds_b) / (float)R + eps);
   for (int d = threadIdx.x; d < QR; d += ROW_BLOCK)
     Act<T>::st(cq + t * QR + d, Act<T>::ld(x + d) * rq * wq[d]);
+  for (int h = threadIdx.x; h < H; h += ROW_BLOCK)
+    gate[t * H + h] = sigmoid_f32(Act<T>::ld(x + QR + R + RD + h));
+  if (cache == nullptr) return;
+  const float rc = 1.0f / sqrtf(row_block_sum(sc, lds_b) / (float)R + eps);
   T* crow = cache + (int64_t)slot_mapping[t] * (R + RD);
   for (int d = threadIdx.x; d < R; d += ROW_BLOCK)
     Act<T>::st(crow + d, Act<T>::ld(x + QR + d) * rc * wc[d]);
   const float pos = (float)positions[t];
   const T* kr = x + QR + R;
   for (int i = threadIdx.x; i < n_pairs; i += ROW_BLOCK) {
-    const float u = Act<T>::ld(kr + 2 * i), v = Act<T>::ld(kr + 2 * i + 1);
+    int a, b;
+    rotary_pair_index(half, i, n_pairs, a, b);
+    const float u = Act<T>::ld(kr + a), v = Act<T>::ld(kr + b);
     float s, c;
     sincosf(pos * inv_freq[i], &s, &c);
-    Act<T>::st(crow + R + 2 * i, u * c - v * s);
-    Act<T>::st(crow + R + 2 * i + 1, v * c + u * s);
+    s *= mag;
+    c *= mag;
+    Act<T>::st(crow + R + a, u * c - v * s);
+    Act<T>::st(crow + R + b, v * c + u * s);
   }
   for (int d = 2 * n_pairs + threadIdx.x; d < RD; d += ROW_BLOCK)
     crow[R + d] = kr[d];
-  for (int h = threadIdx.x; h < H; h += ROW_BLOCK)
-    gate[t * H + h] = sigmoid_f32(Act<T>::ld(x + QR + R + RD + h));
 }
 
 void latent_down_post(torch::Tensor cq, torch::Tensor gate, torch::Tensor down,
                       torch::Tensor positions, torch::Tensor slot_mapping,
-                      torch::Tensor cache, torch::Tensor qnorm_w,
-                      torch::Tensor kvnorm_w, torch::Tensor inv_freq,
-                      double eps, int64_t q_rank, int64_t kv_rank,
-                      int64_t rot_dim, int64_t heads) {
+                      c10::optional<torch::Tensor> cache,
+                      torch::Tensor qnorm_w,
+                      c10::optional<torch::Tensor> kvnorm_w,
+                      torch::Tensor inv_freq, double eps, int64_t q_rank,
+                      int64_t kv_rank, int64_t rot_dim, int64_t heads,
+                      bool half, double mag) {
   const int T = down.size(0);
+  const bool owns = cache.has_value();
+  const int64_t R = owns ? kv_rank : 0, RD = owns ? rot_dim : 0;
   TORCH_CHECK(down.is_cuda() && down.dim() == 2 && down.stride(1) == 1);
-  TORCH_CHECK(down.size(1) == q_rank + kv_rank + rot_dim + heads);
-  TORCH_CHECK(cache.is_contiguous() && cache.dim() == 3 &&
-              cache.size(2) == kv_rank + rot_dim &&
-              cache.dtype() == down.dtype());
+  TORCH_CHECK(down.size(1) == q_rank + R + RD + heads);
+  if (owns) {
+    TORCH_CHECK(cache->is_contiguous() && cache->dim() == 3 &&
+                cache->size(2) == R + RD && cache->dtype() == down.dtype());
+    TORCH_CHECK(kvnorm_w.has_value() &&
+                kvnorm_w->dtype() == torch::kFloat32 &&
+                kvnorm_w->numel() == R);
+  }
   TORCH_CHECK(cq.is_contiguous() && cq.dtype() == down.dtype() &&
               cq.size(0) == T && cq.size(1) == q_rank);
   TORCH_CHECK(gate.is_contiguous() && gate.dtype() == torch::kFloat32 &&
@@ -156,8 +179,6 @@ void latent_down_post(torch::Tensor cq, torch::Tensor gate, torch::Tensor down,
               slot_mapping.numel() == T);
   TORCH_CHECK(qnorm_w.dtype() == torch::kFloat32 &&
               qnorm_w.numel() == q_rank);
-  TORCH_CHECK(kvnorm_w.dtype() == torch::kFloat32 &&
-              kvnorm_w.numel() == kv_rank);
   TORCH_CHECK(inv_freq.dtype() == torch::kFloat32 &&
               2 * inv_freq.numel() <= rot_dim);
   if (T == 0) return;
@@ -168,53 +189,66 @@ void latent_down_post(torch::Tensor cq, torch::Tensor gate, torch::Tensor down,
         (act_t*)cq.data_ptr(), (float*)gate.data_ptr(),
         (const act_t*)down.data_ptr(), (int64_t)down.stride(0),
         (const int32_t*)positions.data_ptr(),
-        (const int32_t*)slot_mapping.data_ptr(), (act_t*)cache.data_ptr(),
-        (const float*)qnorm_w.data_ptr(), (const float*)kvnorm_w.data_ptr(),
-        (const float*)inv_freq.data_ptr(), (int)inv_freq.numel(), (float)eps,
-        (int)q_rank, (int)kv_rank, (int)rot_dim, (int)heads);
+        (const int32_t*)slot_mapping.data_ptr(),
+        owns ? (act_t*)cache->data_ptr() : nullptr,
+        (const float*)qnorm_w.data_ptr(),
+        owns ? (const float*)kvnorm_w->data_ptr() : nullptr,
+        (const float*)inv_freq.data_ptr(),
+        owns ? (int)inv_freq.numel() : 0, half, (float)mag, (float)eps,
+        (int)q_rank, (int)R, (int)RD, (int)heads);
   });
   HIP_CHECK_KERNEL();
 }
 
 // ---------------------------------------------------------------------------
+// one block per token row: its cos / sin are evaluated once (LDS) and
+// shared by all heads
 template <typename T>
-__global__ void rope_pairs_kernel(T* __restrict__ x, int64_t s0, int64_t s1,
-                                  const int32_t* __restrict__ positions,
-                                  const float* __restrict__ inv_freq,
-                                  int n_pairs, int H, int offset,
-                                  int64_t total) {
-  const int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
-  if (i >= total) return;
-  const int p = (int)(i % n_pairs);
-  const int h = (int)((i / n_pairs) % H);
-  const int64_t t = i / ((int64_t)n_pairs * H);
-  T* e = x + t * s0 + h * s1 + offset + 2 * p;
-  const float u = Act<T>::ld(e), v = Act<T>::ld(e + 1);
-  float s, c;
-  sincosf((float)positions[t] * inv_freq[p], &s, &c);
-  Act<T>::st(e, u * c - v * s);
-  Act<T>::st(e + 1, v * c + u * s);
+__global__ __launch_bounds__(ROW_BLOCK) void rope_pairs_kernel(
+    T* __restrict__ x, int64_t s0, int64_t s1,
+    const int32_t* __restrict__ positions, const float* __restrict__ inv_freq,
+    int n_pairs, int H, int offset, bool half, float mag) {
+  extern __shared__ float rope_cs[];
+  const int64_t t = blockIdx.x;
+  const float pos = (float)positions[t];
+  for (int i = threadIdx.x; i < n_pairs; i += ROW_BLOCK) {
+    float s, c;
+    sincosf(pos * inv_freq[i], &s, &c);
+    rope_cs[i] = c * mag;
+    rope_cs[n_pairs + i] = s * mag;
+  }
+  __syncthreads();
+  for (int i = threadIdx.x; i < n_pairs * H; i += ROW_BLOCK) {
+    const int p = i % n_pairs, h = i / n_pairs;
+    int a, b;
+    rotary_pair_index(half, p, n_pairs, a, b);
+    T* e = x + t * s0 + h * s1 + offset;
+    const float u = Act<T>::ld(e + a), v = Act<T>::ld(e + b);
+    const float c = rope_cs[p], s = rope_cs[n_pairs + p];
+    Act<T>::st(e + a, u * c - v * s);
+    Act<T>::st(e + b, v * c + u * s);
+  }
 }
 
 void rope_pairs(torch::Tensor x, torch::Tensor positions,
-                torch::Tensor inv_freq, int64_t offset) {
+                torch::Tensor inv_freq, int64_t offset, bool half,
+                double mag) {
   TORCH_CHECK(x.is_cuda() && x.dim() == 3 && x.stride(2) == 1);
   const int T = x.size(0), H = x.size(1);
   const int n_pairs = inv_freq.numel();
   TORCH_CHECK(offset >= 0 && offset + 2 * n_pairs <= x.size(2));
   TORCH_CHECK(positions.dtype() == torch::kInt32 && positions.numel() == T);
-  TORCH_CHECK(inv_freq.dtype() == torch::kFloat32);
-  const int64_t total = (int64_t)T * H * n_pairs;
-  if (total == 0) return;
+  TORCH_CHECK(inv_freq.dtype() == torch::kFloat32 && n_pairs <= 4096);
+  if (T == 0 || H == 0 || n_pairs == 0) return;
   hipStream_t stream = at::cuda::getCurrentCUDAStream();
   IGW_DISPATCH_ACT(x, {
-    hipLaunchKernelGGL((rope_pairs_kernel<act_t>),
-                       dim3((total + 255) / 256), dim3(256), 0, stream,
+    hipLaunchKernelGGL((rope_pairs_kernel<act_t>), dim3(T), dim3(ROW_BLOCK),
+                       (size_t)(2 * n_pairs) * sizeof(float), stream,
                        (act_t*)x.data_ptr(), (int64_t)x.stride(0),
                        (int64_t)x.stride(1),
                        (const int32_t*)positions.data_ptr(),
                        (const float*)inv_freq.data_ptr(), n_pairs, H,
-                       (int)offset, total);
+                       (int)offset, half, (float)mag);
   });
   HIP_CHECK_KERNEL();
 }

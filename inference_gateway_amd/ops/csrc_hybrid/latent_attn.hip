@@ -10,7 +10,9 @@
 //
 // where the softmax denominator additionally holds exp(sink_h): the sink is
 // folded in as the INITIAL state of the online softmax (running max =
-// sink, running sum = 1, accumulator = 0), i.e. a key with no value.
+// sink, running sum = 1, accumulator = 0), i.e. a key with no value
+// (without sinks the softmax is the ordinary one: empty initial state).
+// With a gate, out[t,h] is multiplied by gate[t,h].
 // Scores, probabilities and the accumulator are fp32.
 //
 // latent_attention_rows: one wave per (row, head); lanes are keys for the
@@ -28,7 +30,8 @@ __global__ __launch_bounds__(64) void latent_attention_rows_kernel(
     const T* __restrict__ cache, const int32_t* __restrict__ block_table,
     int max_blocks, const int32_t* __restrict__ row_seq,
     const int32_t* __restrict__ positions, const float* __restrict__ sink,
-    float scale, int window, int H, int R, int RD, int block_size) {
+    const float* __restrict__ gate, float scale, int window, int H, int R,
+    int RD, int block_size) {
   extern __shared__ float lds[];
   float* q = lds;                      // [R + RD], pre-scaled
   float* p_lds = lds + R + RD;         // [64]
@@ -43,7 +46,7 @@ __global__ __launch_bounds__(64) void latent_attention_rows_kernel(
   for (int d = lane; d < RD; d += 64)
     q[R + d] = Act<T>::ld(q_rot + t * qr_s0 + h * qr_s1 + d) * scale;
   __syncthreads();
-  float m = sink[h], l = 1.0f;
+  float m = sink ? sink[h] : -INFINITY, l = sink ? 1.0f : 0.0f;
   float acc[NACC];
 #pragma unroll
   for (int i = 0; i < NACC; ++i) acc[i] = 0.0f;
@@ -81,7 +84,7 @@ __global__ __launch_bounds__(64) void latent_attention_rows_kernel(
       }
     }
   }
-  const float inv = 1.0f / l;
+  const float inv = (gate ? gate[(int64_t)t * H + h] : 1.0f) / l;
   T* o = out + ((int64_t)t * H + h) * R;
 #pragma unroll
   for (int i = 0; i < NACC; ++i) {
@@ -93,8 +96,9 @@ __global__ __launch_bounds__(64) void latent_attention_rows_kernel(
 void latent_attention(torch::Tensor out, torch::Tensor q_abs,
                       torch::Tensor q_rot, torch::Tensor cache,
                       torch::Tensor block_table, torch::Tensor row_seq,
-                      torch::Tensor positions, torch::Tensor sink,
-                      double scale, int64_t window) {
+                      torch::Tensor positions,
+                      c10::optional<torch::Tensor> sink, double scale,
+                      int64_t window, c10::optional<torch::Tensor> gate) {
   TORCH_CHECK(q_abs.is_cuda() && q_abs.dim() == 3 && q_abs.stride(2) == 1);
   TORCH_CHECK(q_rot.dim() == 3 && q_rot.stride(2) == 1 &&
               q_rot.dtype() == q_abs.dtype());
@@ -109,7 +113,7 @@ void latent_attention(torch::Tensor out, torch::Tensor q_abs,
               block_table.is_contiguous() && block_table.dim() == 2);
   TORCH_CHECK(row_seq.dtype() == torch::kInt32 && row_seq.numel() == T);
   TORCH_CHECK(positions.dtype() == torch::kInt32 && positions.numel() == T);
-  TORCH_CHECK(sink.dtype() == torch::kFloat32 && sink.numel() == H);
+  check_head_vectors(sink, gate, T, H);
   TORCH_CHECK(R <= 1024, "latent width above 1024 is not supported");
   if (T == 0) return;
   hipStream_t stream = at::cuda::getCurrentCUDAStream();
@@ -124,7 +128,9 @@ void latent_attention(torch::Tensor out, torch::Tensor q_abs,
       (int64_t)q_rot.stride(1), (const act_t*)cache.data_ptr(),               \
       (const int32_t*)block_table.data_ptr(), (int)block_table.size(1),       \
       (const int32_t*)row_seq.data_ptr(),                                     \
-      (const int32_t*)positions.data_ptr(), (const float*)sink.data_ptr(),    \
+      (const int32_t*)positions.data_ptr(),                                   \
+      sink.has_value() ? (const float*)sink->data_ptr() : nullptr,            \
+      gate.has_value() ? (const float*)gate->data_ptr() : nullptr,            \
       (float)scale, (int)window, H, R, RD, (int)cache.size(1))
   IGW_DISPATCH_ACT(q_abs, {
     if (nacc <= 1) LAUNCH_ROWS(1);

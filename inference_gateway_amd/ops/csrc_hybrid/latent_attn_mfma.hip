@@ -11,8 +11,8 @@
 // Per key tile, per wave (16 of the 64 pairs):
 //   S  = Q . K^T        mfma 16x16x32 bf16, Q fragments held in registers,
 //                       K tile row-major in LDS
-//   online softmax in fp32 registers; the running max starts at the head's
-//   sink and the running sum at 1 (the sink is a key without a value)
+//   online softmax in fp32 registers; with a sink the running max starts
+//   at the head's sink and the running sum at 1 (a key without a value)
 //   O += P . C          P through a per-wave LDS tile (C layout -> A
 //                       layout), latents staged TRANSPOSED in LDS
 // Two workgroups per compute unit are requested for the smaller register
@@ -41,8 +41,8 @@ __global__ __launch_bounds__(NW * 64, ((NW == 4 && KS <= 10) ? 2 : 1)) void late
     const int32_t* __restrict__ row_seq, const int32_t* __restrict__ positions,
     const int32_t* __restrict__ tile_row0,
     const int32_t* __restrict__ tile_nrows, const float* __restrict__ sink,
-    float scale, int window, int H, int R, int RD, int block_size, int HB,
-    bool qvec) {
+    const float* __restrict__ gate, float scale, int window, int H, int R,
+    int RD, int block_size, int HB, bool qvec) {
   extern __shared__ __attribute__((aligned(16))) uint16_t la_smem[];
   const int CW = R + RD;
   const int ks_n = (CW + 31) / 32;          // 32-wide steps actually used
@@ -124,10 +124,11 @@ __global__ __launch_bounds__(NW * 64, ((NW == 4 && KS <= 10) ? 2 : 1)) void late
     const int r = m / HB, hh = m % HB;
     const bool ok = r < nrows && h0 + hh < H;
     rpos[r4] = ok ? p0 + r : -1;           // -1: sees no key
-    // later splits start empty: a finite "minus infinity" keeps the
-    // rescaling factors well defined
-    m_run[r4] = !ok ? 0.0f : split == 0 ? sink[h0 + hh] : -1e30f;
-    l_run[r4] = split == 0 ? 1.0f : 0.0f;
+    // later splits, and rows without a sink, start empty: a finite "minus
+    // infinity" keeps the rescaling factors well defined
+    const bool seeded = sink && split == 0;
+    m_run[r4] = !ok ? 0.0f : seeded ? sink[h0 + hh] : -1e30f;
+    l_run[r4] = seeded ? 1.0f : 0.0f;
   }
   float4v acc_o[NT];
 #pragma unroll
@@ -272,7 +273,7 @@ __global__ __launch_bounds__(NW * 64, ((NW == 4 && KS <= 10) ? 2 : 1)) void late
     const int r = m / HB, hh = m % HB;
     const int64_t pair = (int64_t)(row0 + r) * H + h0 + hh;
     if (nsplit == 1) {
-      const float inv = 1.0f / l_run[r4];
+      const float inv = (gate ? gate[pair] : 1.0f) / l_run[r4];
       uint16_t* o = out + pair * R;
 #pragma unroll
       for (int nt = 0; nt < NT; ++nt) {
@@ -299,7 +300,8 @@ __global__ __launch_bounds__(NW * 64, ((NW == 4 && KS <= 10) ? 2 : 1)) void late
 // sum_z l_z e^(m_z - M)
 __global__ __launch_bounds__(64) void latent_attention_merge_kernel(
     uint16_t* __restrict__ out, const float* __restrict__ part_o,
-    const float* __restrict__ part_ml, int nsplit, int64_t pairs, int R) {
+    const float* __restrict__ part_ml, const float* __restrict__ gate,
+    int nsplit, int64_t pairs, int R) {
   const int64_t pair = blockIdx.x;
   float M = -INFINITY;
   for (int z = 0; z < nsplit; ++z)
@@ -308,7 +310,7 @@ __global__ __launch_bounds__(64) void latent_attention_merge_kernel(
   for (int z = 0; z < nsplit; ++z)
     den += part_ml[2 * (z * pairs + pair) + 1] *
            expf(part_ml[2 * (z * pairs + pair)] - M);
-  const float inv = 1.0f / den;
+  const float inv = (gate ? gate[pair] : 1.0f) / den;
   for (int d = threadIdx.x; d < R; d += 64) {
     float acc = 0.0f;
     for (int z = 0; z < nsplit; ++z)
@@ -334,8 +336,10 @@ bool latent_attention_mfma(torch::Tensor out, torch::Tensor q_abs,
                            torch::Tensor q_rot, torch::Tensor cache,
                            torch::Tensor block_table, torch::Tensor row_seq,
                            torch::Tensor positions, torch::Tensor tile_row0,
-                           torch::Tensor tile_nrows, torch::Tensor sink,
-                           double scale, int64_t window, int64_t max_keys) {
+                           torch::Tensor tile_nrows,
+                           c10::optional<torch::Tensor> sink, double scale,
+                           int64_t window, int64_t max_keys,
+                           c10::optional<torch::Tensor> gate) {
   TORCH_CHECK(q_abs.is_cuda() && q_abs.dim() == 3 && q_abs.stride(2) == 1 &&
               q_abs.dtype() == torch::kBFloat16);
   TORCH_CHECK(q_rot.dim() == 3 && q_rot.stride(2) == 1 &&
@@ -351,7 +355,7 @@ bool latent_attention_mfma(torch::Tensor out, torch::Tensor q_abs,
               block_table.is_contiguous() && block_table.dim() == 2);
   TORCH_CHECK(row_seq.dtype() == torch::kInt32 && row_seq.numel() == T);
   TORCH_CHECK(positions.dtype() == torch::kInt32 && positions.numel() == T);
-  TORCH_CHECK(sink.dtype() == torch::kFloat32 && sink.numel() == H);
+  check_head_vectors(sink, gate, T, H);
   const int ntiles = tile_row0.numel();
   TORCH_CHECK(tile_row0.dtype() == torch::kInt32 &&
               tile_nrows.dtype() == torch::kInt32 &&
@@ -400,6 +404,8 @@ bool latent_attention_mfma(torch::Tensor out, torch::Tensor q_abs,
     part_ml = torch::empty({nsplit, (int64_t)T * H, 2}, f32);
   }
   dim3 grid(ntiles, hgroups, nsplit);
+  const float* gate_p =
+      gate.has_value() ? (const float*)gate->data_ptr() : nullptr;
   // 16-byte query loads need aligned rows on both query tensors
   const bool qvec =
       R % 8 == 0 && RD % 8 == 0 && q_abs.stride(0) % 8 == 0 &&
@@ -426,7 +432,9 @@ bool latent_attention_mfma(torch::Tensor out, torch::Tensor q_abs,
         (const int32_t*)row_seq.data_ptr(),                                   \
         (const int32_t*)positions.data_ptr(),                                 \
         (const int32_t*)tile_row0.data_ptr(),                                 \
-        (const int32_t*)tile_nrows.data_ptr(), (const float*)sink.data_ptr(), \
+        (const int32_t*)tile_nrows.data_ptr(),                                \
+        sink.has_value() ? (const float*)sink->data_ptr() : nullptr,          \
+        gate_p,                                                               \
         (float)scale, (int)window, H, R, RD, (int)cache.size(1), HB, qvec);   \
   } while (0)
 #define LAUNCH_LA(KSV, NTV)                                                   \
@@ -450,7 +458,7 @@ bool latent_attention_mfma(torch::Tensor out, torch::Tensor q_abs,
     hipLaunchKernelGGL(latent_attention_merge_kernel, dim3((int64_t)T * H),
                        dim3(64), 0, stream, (uint16_t*)out.data_ptr(),
                        (const float*)part_o.data_ptr(),
-                       (const float*)part_ml.data_ptr(), nsplit,
+                       (const float*)part_ml.data_ptr(), gate_p, nsplit,
                        (int64_t)T * H, R);
     HIP_CHECK_KERNEL();
   }

@@ -6,8 +6,8 @@
 //   qk_norm_append    RMS norm over the WHOLE query block and the whole key
 //                     block of a fused projection, value blend with another
 //                     layer's values, paged append of keys and values
-//   gated_act         (gate | up) -> silu(g) u, or the clamped unit
-//                     g' sigmoid(alpha g') (u' + 1)
+//   gated_act         (gate | up) -> silu(g) u, the clamped unit
+//                     g' sigmoid(alpha g') (u' + 1), or gelu_tanh(g) u
 //
 // One 256-thread block (4 waves) per token row for the row-wise kernels;
 // all arithmetic fp32, loads/stores in the activation type.
@@ -355,11 +355,15 @@ void qk_norm_append(torch::Tensor q_out, torch::Tensor proj,
 
 // ---------------------------------------------------------------------------
 // MODE 0: silu(g) * u.  MODE 1: g' = min(g, L), u' = clamp(u, -L, L):
-// g' * sigmoid(alpha * g') * (u' + 1).
+// g' * sigmoid(alpha * g') * (u' + 1).  MODE 2: gelu_tanh(g) * u, by
+// (1 + tanh(x)) / 2 = sigmoid(2x).
 template <typename T, int MODE>
 DEVINLINE float gated_one(float g, float u, float limit, float alpha) {
   if constexpr (MODE == 0) {
     return g * sigmoid_for<T>(g) * u;
+  } else if constexpr (MODE == 2) {
+    const float x = 1.5957691216057308f * (g + 0.044715f * g * g * g);
+    return g * sigmoid_for<T>(x) * u;
   } else {
     g = fminf(g, limit);
     u = fminf(fmaxf(u, -limit), limit);
@@ -396,7 +400,7 @@ void gated_act(torch::Tensor out, torch::Tensor in, int64_t mode, double limit,
                double alpha) {
   TORCH_CHECK(in.is_cuda() && in.is_contiguous() && out.is_contiguous() &&
               out.dtype() == in.dtype());
-  TORCH_CHECK(mode == 0 || mode == 1, "gated_act: unknown mode");
+  TORCH_CHECK(mode >= 0 && mode <= 2, "gated_act: unknown mode");
   const int F = in.size(-1) / 2;
   TORCH_CHECK(in.size(-1) == 2 * F && out.size(-1) == F &&
               out.numel() * 2 == in.numel());
@@ -415,9 +419,12 @@ void gated_act(torch::Tensor out, torch::Tensor in, int64_t mode, double limit,
     if (mode == 0) {
       if (vec == 4) LAUNCH_GATED(0, 4);
       else LAUNCH_GATED(0, 1);
-    } else {
+    } else if (mode == 1) {
       if (vec == 4) LAUNCH_GATED(1, 4);
       else LAUNCH_GATED(1, 1);
+    } else {
+      if (vec == 4) LAUNCH_GATED(2, 4);
+      else LAUNCH_GATED(2, 1);
     }
   });
 #undef LAUNCH_GATED

@@ -51,7 +51,7 @@ void softcap_attention(torch::Tensor out, torch::Tensor q, torch::Tensor kcache,
                        int64_t temp_every, int64_t window,
                        c10::optional<torch::Tensor> slopes, int64_t chunk,
                        c10::optional<torch::Tensor> sinks,
-                       c10::optional<torch::Tensor> gate);
+                       c10::optional<torch::Tensor> gate, int64_t keep);
 bool softcap_attention_mfma(torch::Tensor out, torch::Tensor q,
                             torch::Tensor kcache, torch::Tensor vcache,
                             torch::Tensor block_table, torch::Tensor seq_cu,
@@ -61,7 +61,7 @@ bool softcap_attention_mfma(torch::Tensor out, torch::Tensor q,
                             int64_t temp_every, int64_t window,
                             c10::optional<torch::Tensor> slopes,
                             int64_t chunk, c10::optional<torch::Tensor> sinks,
-                            c10::optional<torch::Tensor> gate);
+                            c10::optional<torch::Tensor> gate, int64_t keep);
 int64_t softcap_attention_tile_rows();
 void delta_scan(torch::Tensor out, torch::Tensor q, torch::Tensor k,
                 torch::Tensor v, torch::Tensor decay, torch::Tensor beta,
@@ -86,7 +86,8 @@ void moe_group_route(torch::Tensor weights, torch::Tensor idx,
 void add_normed_rmsnorm(torch::Tensor out, torch::Tensor residual,
                         c10::optional<torch::Tensor> delta,
                         c10::optional<torch::Tensor> w_post,
-                        c10::optional<torch::Tensor> w_pre, double eps);
+                        c10::optional<torch::Tensor> w_pre, double eps,
+                        double mult);
 void gelu_mul_rows(torch::Tensor out, torch::Tensor z, torch::Tensor table,
                    torch::Tensor tokens, int64_t col0);
 // csrc_hybrid/parallel_ops.hip, csrc_hybrid/hybrid_ops.hip
@@ -129,7 +130,7 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
         "fp32 residual += two deltas; one RMS statistic, two weighted outputs");
   m.def("relu2", &igw::relu2, "squared ReLU activation");
   m.def("gated_act", &igw::gated_act,
-        "gated activations: silu(g)*u or the clamped (u+1) form");
+        "gated activations: silu(g)*u, the clamped (u+1) form, gelu_tanh(g)*u");
   m.def("delta_scan", &igw::delta_scan,
         "gated delta-rule memory recurrence, state columns in registers");
   m.def("decay_beta_gates", &igw::decay_beta_gates,
@@ -139,7 +140,7 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("moe_group_route", &igw::moe_group_route,
         "sigmoid router with a choice correction and expert groups");
   m.def("add_normed_rmsnorm", &igw::add_normed_rmsnorm,
-        "fp32 residual += RMS-normed delta; RMS norm of the sum");
+        "fp32 residual += scaled RMS-normed delta; RMS norm of the sum");
   m.def("gelu_mul_rows", &igw::gelu_mul_rows,
         "gelu_tanh(z) times a slice of a table row gathered by token");
 }

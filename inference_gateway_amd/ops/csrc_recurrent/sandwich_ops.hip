@@ -1,7 +1,7 @@
 // Row kernels of a sandwich-norm layer (an RMS norm before AND after every
 // sublayer) on an fp32 residual stream (gfx950):
 //
-//   add_normed_rmsnorm   residual += rmsnorm(delta) * w_post   (in place)
+//   add_normed_rmsnorm   residual += mult * rmsnorm(delta) * w_post (in place)
 //                        out = rmsnorm(residual) * w_pre, or the residual
 //                        itself in the activation type when w_pre is absent
 //   gelu_mul_rows        gelu_tanh(z) * table[token, col0 : col0 + W]
@@ -16,7 +16,7 @@ __global__ __launch_bounds__(256) void add_normed_rmsnorm_kernel(
     TO* __restrict__ out, float* __restrict__ residual,
     const TD* __restrict__ delta, int64_t delta_rs,
     const float* __restrict__ w_post, const float* __restrict__ w_pre, int D,
-    float eps) {
+    float eps, float mult) {
   __shared__ float red[8];
   const int t = blockIdx.x, tid = threadIdx.x;
   float* res = residual + (int64_t)t * D;
@@ -30,7 +30,7 @@ __global__ __launch_bounds__(256) void add_normed_rmsnorm_kernel(
       sd += x * x;
     }
     sd = block_reduce_sum<256>(sd, red);
-    const float r1 = 1.0f / sqrtf(sd / (float)D + eps);
+    const float r1 = mult / sqrtf(sd / (float)D + eps);
     __syncthreads();
     for (int d = tid; d < D; d += 256) {
       const float x = res[d] + Act<TD>::ld(dl + d) * r1 * w_post[d];
@@ -56,7 +56,8 @@ __global__ __launch_bounds__(256) void add_normed_rmsnorm_kernel(
 void add_normed_rmsnorm(torch::Tensor out, torch::Tensor residual,
                         c10::optional<torch::Tensor> delta,
                         c10::optional<torch::Tensor> w_post,
-                        c10::optional<torch::Tensor> w_pre, double eps) {
+                        c10::optional<torch::Tensor> w_pre, double eps,
+                        double mult) {
   TORCH_CHECK(residual.is_cuda() && residual.dtype() == torch::kFloat32 &&
               residual.is_contiguous() && residual.dim() == 2);
   const int T = residual.size(0), D = residual.size(1);
@@ -83,7 +84,7 @@ void add_normed_rmsnorm(torch::Tensor out, torch::Tensor residual,
                      (float*)residual.data_ptr(),                             \
                      delta.has_value() ? (const TD*)delta->data_ptr()         \
                                        : nullptr,                             \
-                     drs, wp, wn, D, (float)eps)
+                     drs, wp, wn, D, (float)eps, (float)mult)
   const bool d16 = delta.has_value() &&
                    delta->scalar_type() == torch::kBFloat16;
   if (delta.has_value())

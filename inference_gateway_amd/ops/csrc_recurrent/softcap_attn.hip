@@ -10,10 +10,12 @@
 //
 // lo = max(0, p - window + 1) with a window, 0 without; with chunk > 0 also
 // lo >= floor(p / chunk) * chunk (keys of the row's own position chunk).
+// With keep > 0 the first `keep` keys of the sequence stay visible whatever
+// lo is.
 // With sinks, exp(sink[h]) joins the softmax denominator (a key of that
-// score without a value); with a gate, out[t,h] *= sigmoid(gate[t,h]).  Keys are
-// [blocks, G, block, N], values [blocks, G, block, P]; N and P need not be
-// equal.  Scores, probabilities and the accumulator are fp32.
+// score without a value); with a gate, out[t,h] *= sigmoid(gate[t,h]), one
+// number per value entry or one per head.  Keys are [blocks, G, block, N],
+// values [blocks, G, block, P]; N and P need not be equal.  Scores, probabilities and the accumulator are fp32.
 //
 // softcap_attention_rows: one wave per (row, head); lanes are keys for the
 // scores and value entries for the weighted sum.  Works for any sizes and
@@ -30,9 +32,10 @@ __global__ __launch_bounds__(64) void softcap_attention_rows_kernel(
     const int32_t* __restrict__ block_table, int max_blocks,
     const int32_t* __restrict__ row_seq, const int32_t* __restrict__ positions,
     float scale, float softcap, float temp_coef, int temp_every, int window,
-    const float* __restrict__ slopes, int chunk,
+    const float* __restrict__ slopes, int chunk, int keep,
     const float* __restrict__ sinks, const T* __restrict__ gate,
-    int64_t gate_stride, int H, int G, int N, int P, int block_size) {
+    int64_t gate_stride, int gate_w, int H, int G, int N, int P,
+    int block_size) {
   extern __shared__ float lds[];
   float* ql = lds;                            // [N], pre-scaled
   float* p_lds = lds + N;                     // [64]
@@ -55,9 +58,13 @@ __global__ __launch_bounds__(64) void softcap_attention_rows_kernel(
   float acc[NACC];
 #pragma unroll
   for (int i = 0; i < NACC; ++i) acc[i] = 0.0f;
-  for (int j0 = lo; j0 <= pos; j0 += 64) {
-    const int j = j0 + lane;
-    const bool valid = j <= pos;
+  // visible keys, in order: the kept ones below lo, then [lo, pos]
+  const int kept = min(keep, lo);
+  const int total = kept + pos - lo + 1;
+  for (int i0 = 0; i0 < total; i0 += 64) {
+    const int i = i0 + lane;
+    const bool valid = i < total;
+    const int j = i < kept ? i : lo + i - kept;
     float s = -INFINITY;
     int32_t prow = 0;
     if (valid) {
@@ -80,7 +87,7 @@ __global__ __launch_bounds__(64) void softcap_attention_rows_kernel(
     p_lds[lane] = pr;
     row_lds[lane] = prow;
     __syncthreads();
-    const int n = min(64, pos - j0 + 1);
+    const int n = min(64, total - i0);
     for (int kx = 0; kx < n; ++kx) {
       const float pk = p_lds[kx];
       const T* row = vcache + (int64_t)row_lds[kx] * P;
@@ -96,13 +103,13 @@ __global__ __launch_bounds__(64) void softcap_attention_rows_kernel(
   if (sinks) l += expf(sinks[h] - m);
   const float inv = 1.0f / l;
   T* o = out + ((int64_t)t * H + h) * P;
-  const T* gt = gate ? gate + (int64_t)t * gate_stride + h * P : nullptr;
+  const T* gt = gate ? gate + (int64_t)t * gate_stride + h * gate_w : nullptr;
 #pragma unroll
   for (int i = 0; i < NACC; ++i) {
     const int d = lane + 64 * i;
     if (d < P) {
       float y = acc[i] * inv;
-      if (gt) y *= sigmoid_f32(Act<T>::ld(gt + d));
+      if (gt) y *= sigmoid_f32(Act<T>::ld(gt + (gate_w == 1 ? 0 : d)));
       Act<T>::st(o + d, y);
     }
   }
@@ -115,7 +122,7 @@ void softcap_attention(torch::Tensor out, torch::Tensor q, torch::Tensor kcache,
                        int64_t temp_every, int64_t window,
                        c10::optional<torch::Tensor> slopes, int64_t chunk,
                        c10::optional<torch::Tensor> sinks,
-                       c10::optional<torch::Tensor> gate) {
+                       c10::optional<torch::Tensor> gate, int64_t keep) {
   TORCH_CHECK(q.is_cuda() && q.dim() == 2 && q.stride(1) == 1);
   TORCH_CHECK(kcache.is_contiguous() && kcache.dim() == 4 &&
               vcache.is_contiguous() && vcache.dim() == 4 &&
@@ -133,7 +140,7 @@ void softcap_attention(torch::Tensor out, torch::Tensor q, torch::Tensor kcache,
   TORCH_CHECK(row_seq.dtype() == torch::kInt32 && row_seq.numel() == T);
   TORCH_CHECK(positions.dtype() == torch::kInt32 && positions.numel() == T);
   TORCH_CHECK(P <= 1024, "value width above 1024 is not supported");
-  TORCH_CHECK(temp_every >= 1 && chunk >= 0);
+  TORCH_CHECK(temp_every >= 1 && chunk >= 0 && keep >= 0);
   if (slopes.has_value())
     TORCH_CHECK(slopes->dtype() == torch::kFloat32 &&
                 slopes->is_contiguous() && slopes->numel() == H);
@@ -143,7 +150,8 @@ void softcap_attention(torch::Tensor out, torch::Tensor q, torch::Tensor kcache,
   if (gate.has_value())
     TORCH_CHECK(gate->dtype() == q.dtype() && gate->dim() == 2 &&
                 gate->stride(1) == 1 && gate->size(0) == T &&
-                gate->size(1) == (int64_t)H * P);
+                (gate->size(1) == (int64_t)H * P || gate->size(1) == H));
+  const int gate_w = gate.has_value() ? (int)(gate->size(1) / H) : 1;
   if (T == 0) return;
   hipStream_t stream = at::cuda::getCurrentCUDAStream();
   const size_t shmem = (size_t)(N + 128) * sizeof(float);
@@ -159,10 +167,10 @@ void softcap_attention(torch::Tensor out, torch::Tensor q, torch::Tensor kcache,
       (const int32_t*)positions.data_ptr(), (float)scale, (float)softcap,    \
       (float)temp_coef, (int)temp_every, (int)window,                        \
       slopes.has_value() ? (const float*)slopes->data_ptr() : nullptr,       \
-      (int)chunk,                                                            \
+      (int)chunk, (int)keep,                                                 \
       sinks.has_value() ? (const float*)sinks->data_ptr() : nullptr,         \
       gate.has_value() ? (const act_t*)gate->data_ptr() : nullptr,           \
-      gate.has_value() ? (int64_t)gate->stride(0) : 0, H, G, N, P, bs)
+      gate.has_value() ? (int64_t)gate->stride(0) : 0, gate_w, H, G, N, P, bs)
   IGW_DISPATCH_ACT(q, {
     if (nacc <= 1) LAUNCH_ROWS(1);
     else if (nacc <= 2) LAUNCH_ROWS(2);

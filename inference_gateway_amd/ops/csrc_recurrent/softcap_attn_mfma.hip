@@ -9,11 +9,13 @@
 //     to the template's NP / PP (N, P multiples of 8);
 //   * any page size;
 //   * score = q.k * scale * temp(position), then cap * tanh(. / cap);
-//   * an optional sliding window, an optional restriction to the row's
-//     own chunk of positions, an optional linear distance bias per head
+//   * an optional sliding window (with, optionally, the first tokens of the
+//     sequence kept in sight: the tiles between them and the window are
+//     never fetched), an optional restriction to the row's own chunk of
+//     positions, an optional linear distance bias per head
 //     (slope * (row position - key position) is taken off the score), an
 //     optional sink term per head in the softmax denominator and an
-//     optional sigmoid output gate;
+//     optional sigmoid output gate (per value entry or per head);
 //   * two row maps.  Prompt tiles: rows are 64 consecutive tokens of one
 //     head (grid = tiles x heads).  Decoded rows (HEADS_ROWS): the rows of
 //     a tile are the query heads that share one key/value head, so every
@@ -62,9 +64,9 @@ __global__ __launch_bounds__(256, 2) void softcap_attention_mfma_kernel(
     const int32_t* __restrict__ tile_seq, const int32_t* __restrict__ tile_off,
     int H, int G, int N, int P, int BS, float scale, float softcap,
     float temp_coef, int temp_every, int window,
-    const float* __restrict__ slopes, int chunk,
+    const float* __restrict__ slopes, int chunk, int keep,
     const float* __restrict__ sinks, const uint16_t* __restrict__ gate,
-    int64_t gate_rs) {
+    int64_t gate_rs, int gate_w) {
   constexpr int BM = SA_BM, BN = SA_BN;
   constexpr int KROWB = NP * 2;          // bytes per staged Q / K row
   // K tile (shared with the Q staging) | V^T tile | per-wave P tiles
@@ -159,6 +161,14 @@ __global__ __launch_bounds__(256, 2) void softcap_attention_mfma_kernel(
   int kfirst = window > 0 ? max(0, P0 + qoff - window + 1) : 0;
   if (chunk > 0) kfirst = max(kfirst, (P0 + qoff) / chunk * chunk);
   kfirst = kfirst / BN * BN;
+  // kept first keys: their tiles come first, then the loop jumps to the
+  // window
+  const int kkept = keep > 0 ? min((keep + BN - 1) / BN * BN, kfirst) : 0;
+  const int kbegin = kkept > 0 ? 0 : kfirst;
+  auto next_tile = [&](int kb) {
+    kb += BN;
+    return kb >= kkept && kb < kfirst ? kfirst : kb;
+  };
 
   // the next K/V tile travels in registers while the current one is used
   // (a second tile in flight costs more in occupancy than it hides)
@@ -196,9 +206,9 @@ __global__ __launch_bounds__(256, 2) void softcap_attention_mfma_kernel(
       }
     }
   };
-  if (kfirst < kend) fetch(kfirst);
+  if (kbegin < kend) fetch(kbegin);
 
-  for (int kbase = kfirst; kbase < kend; kbase += BN) {
+  for (int kbase = kbegin; kbase < kend; kbase = next_tile(kbase)) {
     __syncthreads();
 #pragma unroll
     for (int it = 0; it < KIT; ++it) {
@@ -221,7 +231,7 @@ __global__ __launch_bounds__(256, 2) void softcap_attention_mfma_kernel(
             vreg[it].v[e];
     }
     __syncthreads();
-    if (kbase + BN < kend) fetch(kbase + BN);
+    if (next_tile(kbase) < kend) fetch(next_tile(kbase));
     // a wave none of whose 16 rows exists only helps with the staging
     if (wave * 16 >= nrows) continue;
 
@@ -251,7 +261,8 @@ __global__ __launch_bounds__(256, 2) void softcap_attention_mfma_kernel(
         float s = acc_s[nt][r] * rscale[r];
         if (softcap > 0.0f) s = softcap * tanh_fast(s * inv_cap);
         s -= slope[r] * (float)(qpos[r] - kpos);
-        if (kpos > qpos[r] || kpos >= KVL || kpos < lo) s = -INFINITY;
+        if (kpos > qpos[r] || kpos >= KVL || (kpos < lo && kpos >= keep))
+          s = -INFINITY;
         acc_s[nt][r] = s;
         mx = fmaxf(mx, s);
       }
@@ -310,13 +321,13 @@ __global__ __launch_bounds__(256, 2) void softcap_attention_mfma_kernel(
     const float lsum = sinks ? l[r] + __expf(sinks[head] - m[r]) : l[r];
     const float inv = 1.0f / lsum;
     uint16_t* o = out + (tok * H + head) * P;
-    const uint16_t* gt = gate ? gate + tok * gate_rs + head * P : nullptr;
+    const uint16_t* gt = gate ? gate + tok * gate_rs + head * gate_w : nullptr;
 #pragma unroll
     for (int nt = 0; nt < PP / 16; ++nt) {
       const int c = nt * 16 + ccol;
       if (c < P) {
         float y = acc_o[nt][r] * inv;
-        if (gt) y *= sigmoid_fast(bf16_to_f32(gt[c]));
+        if (gt) y *= sigmoid_fast(bf16_to_f32(gt[gate_w == 1 ? 0 : c]));
         o[c] = f32_to_bf16(y);
       }
     }
@@ -337,7 +348,7 @@ bool softcap_attention_mfma(torch::Tensor out, torch::Tensor q,
                             int64_t temp_every, int64_t window,
                             c10::optional<torch::Tensor> slopes,
                             int64_t chunk, c10::optional<torch::Tensor> sinks,
-                            c10::optional<torch::Tensor> gate) {
+                            c10::optional<torch::Tensor> gate, int64_t keep) {
   TORCH_CHECK(q.is_cuda() && q.dim() == 2 && q.stride(1) == 1);
   if (q.scalar_type() != torch::kBFloat16) return false;
   TORCH_CHECK(kcache.is_contiguous() && kcache.dim() == 4 &&
@@ -364,7 +375,7 @@ bool softcap_attention_mfma(torch::Tensor out, torch::Tensor q,
   TORCH_CHECK(tile_seq.dtype() == torch::kInt32 &&
               tile_off.dtype() == torch::kInt32 &&
               tile_off.numel() == ntile && dec_seq.dtype() == torch::kInt32);
-  TORCH_CHECK(temp_every >= 1 && chunk >= 0);
+  TORCH_CHECK(temp_every >= 1 && chunk >= 0 && keep >= 0);
   if (slopes.has_value())
     TORCH_CHECK(slopes->dtype() == torch::kFloat32 &&
                 slopes->is_contiguous() && slopes->numel() == H);
@@ -374,7 +385,8 @@ bool softcap_attention_mfma(torch::Tensor out, torch::Tensor q,
   if (gate.has_value())
     TORCH_CHECK(gate->dtype() == q.dtype() && gate->dim() == 2 &&
                 gate->stride(1) == 1 && gate->size(0) == T &&
-                gate->size(1) == (int64_t)H * P);
+                (gate->size(1) == (int64_t)H * P || gate->size(1) == H));
+  const int gate_w = gate.has_value() ? (int)(gate->size(1) / H) : 1;
   hipStream_t stream = at::cuda::getCurrentCUDAStream();
 #define LAUNCH_SA(NPV, PPV, HR, GRID, TSEQ)                                   \
   hipLaunchKernelGGL(                                                         \
@@ -388,10 +400,10 @@ bool softcap_attention_mfma(torch::Tensor out, torch::Tensor q,
       H, G, N, P, BS, (float)scale, (float)softcap, (float)temp_coef,         \
       (int)temp_every, (int)window,                                           \
       slopes.has_value() ? (const float*)slopes->data_ptr() : nullptr,        \
-      (int)chunk,                                                             \
+      (int)chunk, (int)keep,                                                  \
       sinks.has_value() ? (const float*)sinks->data_ptr() : nullptr,          \
       gate.has_value() ? (const uint16_t*)gate->data_ptr() : nullptr,         \
-      gate.has_value() ? (int64_t)gate->stride(0) : 0)
+      gate.has_value() ? (int64_t)gate->stride(0) : 0, gate_w)
 #define LAUNCH_SA_SIZES(HR, GRID, TSEQ)                                       \
   do {                                                                        \
     if (N <= 64 && P <= 64) LAUNCH_SA(64, 64, HR, GRID, TSEQ);                \

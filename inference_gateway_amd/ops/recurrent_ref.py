@@ -210,16 +210,16 @@ def append_paged_kv_ref(k, v, kcache, vcache, slot_mapping):
 def softcap_attention_ref(q, kcache, vcache, block_table, row_seq,
                           positions, scale, softcap, temp_coef, temp_every,
                           window, slopes=None, chunk=0, sinks=None,
-                          gate=None):
+                          gate=None, keep=0):
     """Causal softmax attention of every row against its sequence's
     paged keys 0..position (the last `window` of them when window > 0).
     score = (q . k) * scale * temp(p), temp(p) = 1 + temp_coef *
     ln(floor((p + 1) / temp_every) + 1); then softcap * tanh(score /
     softcap) when softcap > 0.  slopes [H]: slope_h * (p - j) is taken
     off the score of key j.  chunk > 0: only keys from floor(p / chunk) *
-    chunk on.  sinks [H]: exp(sink_h) joins the softmax denominator (a
+    chunk on.  keep > 0: the first `keep` keys stay visible.  sinks [H]: exp(sink_h) joins the softmax denominator (a
     key with that score and no value).  gate [T, H*P]: the result is
-    multiplied by sigmoid(gate).  q [T, H*N] -> [T, H*P]."""
+    multiplied by sigmoid(gate) (gate [T, H]: one per head).  q [T, H*N] -> [T, H*P]."""
     nb, G, bs, N = kcache.shape
     P = vcache.shape[3]
     T = q.shape[0]
@@ -235,6 +235,8 @@ def softcap_attention_ref(q, kcache, vcache, block_table, row_seq,
         if chunk > 0:
             lo = max(lo, p // chunk * chunk)
         j = torch.arange(lo, p + 1, device=q.device)
+        if min(keep, lo) > 0:
+            j = torch.cat([torch.arange(min(keep, lo), device=q.device), j])
         blocks = block_table[seq_l[t]].to(torch.int64)[j // bs]
         kk = kcache[blocks, :, j % bs].float()      # [n, G, N]
         vv = vcache[blocks, :, j % bs].float()      # [n, G, P]
@@ -251,10 +253,9 @@ def softcap_attention_ref(q, kcache, vcache, block_table, row_seq,
         else:
             w = torch.softmax(s, -1)
         out[t] = torch.einsum("hj,jhp->hp", w, vv)
-    out = out.reshape(T, H * P)
     if gate is not None:
-        out = out * torch.sigmoid(gate.float())
-    return out.to(q.dtype)
+        out = out * torch.sigmoid(gate.float()).view(T, H, -1)
+    return out.reshape(T, H * P).to(q.dtype)
 
 
 def qk_norm_rope_append_ref(proj, positions, slot_mapping, kcache, vcache,
@@ -362,14 +363,15 @@ def moe_group_route_ref(logits, correction, top, groups, keep):
     return s.gather(1, idx), idx.to(torch.int32)
 
 
-def add_normed_rmsnorm_ref(residual, delta, w_post, w_pre, eps, out_dtype):
-    """residual [T, D] fp32 += rmsnorm(delta) * w_post (in place; delta
+def add_normed_rmsnorm_ref(residual, delta, w_post, w_pre, eps, out_dtype,
+                           mult=1.0):
+    """residual [T, D] fp32 += mult * rmsnorm(delta) * w_post (in place; delta
     None = nothing added); returns rmsnorm(residual) * w_pre in
     out_dtype, or the residual itself in out_dtype when w_pre is None."""
     if delta is not None:
         d = delta.float()
-        residual += d * torch.rsqrt((d * d).mean(-1, keepdim=True)
-                                    + eps) * w_post
+        residual += d * (mult * torch.rsqrt(
+            (d * d).mean(-1, keepdim=True) + eps)) * w_post
     if w_pre is None:
         return residual.to(out_dtype)
     return (residual * torch.rsqrt((residual * residual).mean(

@@ -360,29 +360,50 @@ def _rope_pairs(x, positions, inv_freq):
     return torch.stack((u * c - v * s, v * c + u * s), -1).flatten(-2)
 
 
-def rope_pairs_ref(x, positions, inv_freq, offset):
+def _rope_halves(x, positions, inv_freq, mag):
+    """x [T, (H,) 2n]: entry i paired with entry i + n."""
+    ang = positions.float()[:, None] * inv_freq[None, :]
+    if x.dim() == 3:
+        ang = ang[:, None]
+    c, s = torch.cos(ang) * mag, torch.sin(ang) * mag
+    u, v = x.chunk(2, -1)
+    return torch.cat([u * c - v * s, v * c + u * s], -1)
+
+
+def _rotate(x, positions, inv_freq, half, mag):
+    """2*len(inv_freq) entries in either pair layout."""
+    if half:
+        return _rope_halves(x, positions, inv_freq, mag)
+    return _rope_pairs(x, positions, inv_freq) * mag
+
+
+def rope_pairs_ref(x, positions, inv_freq, offset, half=False, mag=1.0):
     """In place on x[..., offset : offset + 2*len(inv_freq)]."""
     n2 = 2 * inv_freq.numel()
     part = x[..., offset:offset + n2]
-    part.copy_(_rope_pairs(part.float(), positions, inv_freq).to(x.dtype))
+    part.copy_(_rotate(part.float(), positions, inv_freq, half,
+                       mag).to(x.dtype))
     return x
 
 
 def latent_down_post_ref(down, positions, slot_mapping, cache, qnorm_w,
                          kvnorm_w, inv_freq, eps, q_rank, kv_rank, rot_dim,
-                         heads):
+                         heads, half=False, mag=1.0):
     """Everything between the fused down projection and the up
     projections: RMS-norm the query latent, RMS-norm the key/value
     latent and write it with the rotated shared key into the paged
-    cache, and squash the per-head output gate."""
+    cache (cache None: no key/value part), and squash the per-head
+    output gate."""
     x = down.float()
     cq = x[:, :q_rank]
     cq = cq * torch.rsqrt((cq * cq).mean(-1, keepdim=True) + eps) * qnorm_w
+    if cache is None:
+        return cq.to(down.dtype), torch.sigmoid(x[:, q_rank:q_rank + heads])
     c = x[:, q_rank:q_rank + kv_rank]
     c = c * torch.rsqrt((c * c).mean(-1, keepdim=True) + eps) * kvnorm_w
     kr = x[:, q_rank + kv_rank:q_rank + kv_rank + rot_dim].clone()
     n2 = 2 * inv_freq.numel()
-    kr[:, :n2] = _rope_pairs(kr[:, :n2], positions, inv_freq)
+    kr[:, :n2] = _rotate(kr[:, :n2], positions, inv_freq, half, mag)
     flat = cache.view(-1, cache.shape[-1])
     flat[slot_mapping.long()] = torch.cat([c, kr], -1).to(cache.dtype)
     gate = torch.sigmoid(x[:, q_rank + kv_rank + rot_dim:
@@ -391,11 +412,12 @@ def latent_down_post_ref(down, positions, slot_mapping, cache, qnorm_w,
 
 
 def latent_attention_ref(q_abs, q_rot, cache, block_table, row_seq,
-                         positions, sink, scale, window):
+                         positions, sink, scale, window, gate=None):
     """Absorbed latent attention over the paged cache.  Row t of head h
     scores key j as (q_abs[t,h] . c_j + q_rot[t,h] . kr_j) * scale for
-    pos-window < j <= pos; the softmax denominator also holds exp(sink_h).
-    Returns the probability-weighted sum of latents [T, H, kv_rank]."""
+    pos-window < j <= pos; the softmax denominator also holds exp(sink_h)
+    (sink None: nothing).  Returns the probability-weighted sum of latents
+    [T, H, kv_rank], times gate [T, H] when given."""
     T, H, R = q_abs.shape
     bs = cache.shape[1]
     out = torch.zeros((T, H, R), dtype=torch.float32, device=q_abs.device)
@@ -410,10 +432,16 @@ def latent_attention_ref(q_abs, q_rot, cache, block_table, row_seq,
         bt = block_table[seqs[t]].long()
         rows = flat[bt[j // bs] * bs + j % bs].float()        # [n, R+rd]
         sc = (qa[t] @ rows[:, :R].t() + qr[t] @ rows[:, R:].t()) * scale
-        m = torch.maximum(sc.max(-1).values, sink)            # [H]
+        m = sc.max(-1).values                                 # [H]
+        if sink is not None:
+            m = torch.maximum(m, sink)
         e = torch.exp(sc - m[:, None])
-        den = e.sum(-1) + torch.exp(sink - m)
+        den = e.sum(-1)
+        if sink is not None:
+            den = den + torch.exp(sink - m)
         out[t] = (e @ rows[:, :R]) / den[:, None]
+    if gate is not None:
+        out = out * gate[:, :, None]
     return out.to(q_abs.dtype)
 
 
@@ -541,6 +569,7 @@ def sigmoid_attention_ref(q, kcache, vcache, block_table, row_seq,
 GATED_ACT_SILU = 0       # silu(g) * u
 GATED_ACT_CLAMPED = 1    # min(g, L) * sigmoid(alpha * min(g, L))
                          #   * (clamp(u, -L, L) + 1)
+GATED_ACT_GELU = 2       # gelu_tanh(g) * u
 
 
 def gated_act_ref(gate_up, mode, limit=0.0, alpha=1.0):
@@ -549,6 +578,8 @@ def gated_act_ref(gate_up, mode, limit=0.0, alpha=1.0):
     g, u = gate_up[..., :f].float(), gate_up[..., f:].float()
     if mode == GATED_ACT_SILU:
         y = g * torch.sigmoid(g) * u
+    elif mode == GATED_ACT_GELU:
+        y = torch.nn.functional.gelu(g, approximate="tanh") * u
     else:
         g = torch.clamp(g, max=limit)
         u = torch.clamp(u, min=-limit, max=limit)

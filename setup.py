@@ -33,6 +33,15 @@ REC = ROOT / "inference_gateway_amd" / "ops" / "csrc_recurrent"
 # row kernels (fused add + RMS norm, squared ReLU) its models share
 recurrent_sources = [str(REC / "bindings.cpp")] + _hip_sources(REC) + [str(HYB / "parallel_ops.hip"), str(HYB / "hybrid_ops.hip")]
 
+# the post-norm extension has no kernel sources of its own: it links the
+# attention and row kernels that its models launch
+PN = ROOT / "inference_gateway_amd" / "ops" / "csrc_postnorm"
+postnorm_sources = [str(PN / "bindings.cpp")] + [
+    str(HYB / f) for f in ("hybrid_ops.hip", "latent_attn.hip",
+                           "latent_attn_mfma.hip", "parallel_ops.hip")] + [
+    str(REC / f) for f in ("qk_rope_append.hip", "sandwich_ops.hip",
+                           "softcap_attn.hip", "softcap_attn_mfma.hip")]
+
 # packed-fp32 instruction selection is switched off for all device code
 HIPCC_FLAGS = [
     "-O3",
@@ -51,7 +60,7 @@ def _ext(name, srcs):
     )
 
 
-# IGW_BUILD_EXT=hybrid|kernels|recurrent builds just one extension (a
+# IGW_BUILD_EXT=hybrid|kernels|postnorm|recurrent builds just one extension (a
 # process that serves one model family compiles only what it loads);
 # default: all
 _which = os.environ.get("IGW_BUILD_EXT", "all")
@@ -65,6 +74,9 @@ if _which in ("all", "hybrid"):
 if _which in ("all", "recurrent"):
     ext_modules.append(_ext("inference_gateway_amd.ops._recurrent",
                             recurrent_sources))
+if _which in ("all", "postnorm"):
+    ext_modules.append(_ext("inference_gateway_amd.ops._postnorm",
+                            postnorm_sources))
 
 setup(
     name="inference_gateway_amd_kernels",
