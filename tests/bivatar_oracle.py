@@ -47,18 +47,20 @@ def visible(i, window, keep):
             if not window or i - j < window or j < keep]
 
 
-def window_attention(q, k, v, H, G, scale, window, keep, slopes=None):
+def window_attention(q, k, v, H, G, scale, window, keep, slopes=None,
+                     rows=None):
     """q [T, H, N], k [T, G, N], v [T, G, P]; score = q.k * scale -
-    slope_h (i - j) over the visible j, softmax."""
-    T = q.shape[0]
+    slope_h (i - j) over the visible j, softmax.  rows: only these
+    positions' outputs."""
+    rows = range(q.shape[0]) if rows is None else rows
     slopes = distance_slopes(H) if slopes is None else slopes
-    out = np.zeros((T, H, v.shape[2]))
-    for i in range(T):
+    out = np.zeros((len(rows), H, v.shape[2]))
+    for n, i in enumerate(rows):
         js = np.array(visible(i, window, keep))
         for h in range(H):
             g = h // (H // G)
             s = k[js, g] @ q[i, h] * scale - slopes[h] * (i - js)
-            out[i, h] = softmax(s) @ v[js, g]
+            out[n, h] = softmax(s) @ v[js, g]
     return out
 
 
