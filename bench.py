@@ -87,7 +87,8 @@ def parse_args():
     ap.add_argument("--arch", type=str, default="fedatar",
                     help="design for --arch-compare: fedatar or mekevik "
                          "(each beside Mixtral), feditar (beside "
-                         "Fedatar) or bozolorn (beside Feditar)")
+                         "Fedatar), bozolorn (beside Feditar) or "
+                         "bivatar (beside Fedatar)")
     ap.add_argument("--arch-size", type=str, default="2k",
                     help="layer shape for --arch-compare (2k | 4k)")
     ap.add_argument("--num-gpu-blocks", type=int, default=0,
@@ -520,6 +521,8 @@ def main() -> None:
             import bench_recurrent as bench_hybrid
         elif args.arch == "bozolorn":
             import bench_bozolorn as bench_hybrid
+        elif args.arch == "bivatar":
+            import bench_bivatar as bench_hybrid
         else:
             import bench_hybrid
 

@@ -936,3 +936,24 @@ def test_trace_command(tmp_path):
     assert not (tmp_path / "o" / "1.f32").exists()
     close(g0, ra[[0, 4]], 2e-4)
     close(g2, np.stack([ra[8], rb[3]]), 2e-4)
+
+
+def test_bench_configurations_are_comparable():
+    """The speed comparison runs both models at equal width, head and
+    latent sizes and feed-forward parameters."""
+    root = Path(__file__).resolve().parent.parent
+    sys.path.insert(0, str(root / "tools"))
+    try:
+        import bench_bivatar as bb
+    finally:
+        sys.path.pop(0)
+    for sz in bb.SIZES.values():
+        biv, fed = bb._configs(sz)
+        assert biv.hidden_size == fed.hidden_size == sz["width"]
+        assert biv.num_layers == fed.num_layers
+        assert 3 * biv.layers[0].mlp.ff == 2 * fed.layers[0].mlp.ff
+        a, f = biv.layers[1].mixer, fed.layers[1].mixer
+        for k in ("heads", "dim", "rot_dim", "vdim", "kv_rank", "q_rank",
+                  "window"):
+            assert getattr(a, k) == getattr(f, k)
+        assert biv.layers[3].mixer.kv_from == 1
