@@ -475,17 +475,6 @@ def relu2(z):
     return torch_ref.relu2_ref(z)
 
 
-def gate_heads(v, gate):
-    """v [H, T, vd] (strided ok), gate [T, H] fp32 -> [T, H*vd]."""
-    if v.is_cuda:
-        _require_hybrid()
-        H, T, vd = v.shape
-        out = torch.empty((T, H * vd), dtype=v.dtype, device=v.device)
-        _hybrid.gate_heads(out, v, gate)
-        return out
-    return torch_ref.gate_heads_ref(v, gate)
-
-
 def moe_topk_route(logits, top_k: int, capacity: int = 0,
                    scale: float = 1.0):
     """logits [T, E] fp32 -> (softmax-over-chosen weights [T, K] fp32

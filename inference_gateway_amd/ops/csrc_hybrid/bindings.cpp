@@ -21,7 +21,6 @@ void rope_pairs(torch::Tensor x, torch::Tensor positions,
                 double mag);
 void xielu(torch::Tensor out, torch::Tensor in, torch::Tensor pq);
 void relu2(torch::Tensor out, torch::Tensor in);
-void gate_heads(torch::Tensor out, torch::Tensor v, torch::Tensor gate);
 void moe_topk_route(torch::Tensor weights, torch::Tensor idx,
                     torch::Tensor logits, c10::optional<torch::Tensor> dst,
                     c10::optional<torch::Tensor> counts, int64_t capacity,
@@ -89,8 +88,6 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
         "in-place rotary on a slice of every head, interleaved or half pairs");
   m.def("xielu", &igw::xielu, "xIELU activation");
   m.def("relu2", &igw::relu2, "squared ReLU activation");
-  m.def("gate_heads", &igw::gate_heads,
-        "[H,T,vd] values times [T,H] gates -> [T,H*vd]");
   m.def("moe_topk_route", &igw::moe_topk_route,
         "top-k experts and softmax over the chosen logits");
   m.def("add_rmsnorm_pair", &igw::add_rmsnorm_pair,

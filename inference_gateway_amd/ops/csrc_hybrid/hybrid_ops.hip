@@ -3,11 +3,12 @@
 //   add_layernorm     residual(fp32) += delta; out = LayerNorm(residual)
 //   latent_down_post  RMS-norm the two latents of a fused down projection,
 //                     rotate the shared key, append (latent | key) to the
-//                     paged cache, squash the head gates
-//   rope_pairs        in-place interleaved-pair rotation of a slice of
-//                     every head
+//                     paged cache, squash the head gates (a layer that
+//                     reads another layer's rows has only the query latent
+//                     and the gates)
+//   rope_pairs        in-place rotation of a slice of every head, pairs
+//                     interleaved or half a slice apart
 //   xielu / relu2     feed-forward activations
-//   gate_heads        [H, T, vd] * gate[T, H] -> [T, H*vd]
 //   moe_topk_route    top-k experts + softmax over the chosen logits (times
 //                     a constant)
 //
@@ -312,40 +313,6 @@ void relu2(torch::Tensor out, torch::Tensor in) {
     hipLaunchKernelGGL((relu2_kernel<act_t>), dim3(ew_blocks(n)), dim3(256), 0,
                        stream, (act_t*)out.data_ptr(),
                        (const act_t*)in.data_ptr(), n);
-  });
-  HIP_CHECK_KERNEL();
-}
-
-// ---------------------------------------------------------------------------
-template <typename T>
-__global__ void gate_heads_kernel(T* __restrict__ out, const T* __restrict__ v,
-                                  int64_t sh, int64_t st_,
-                                  const float* __restrict__ gate, int H,
-                                  int VD, int64_t total) {
-  const int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
-  if (i >= total) return;
-  const int d = (int)(i % VD);
-  const int h = (int)((i / VD) % H);
-  const int64_t t = i / ((int64_t)VD * H);
-  Act<T>::st(out + i, Act<T>::ld(v + h * sh + t * st_ + d) * gate[t * H + h]);
-}
-
-void gate_heads(torch::Tensor out, torch::Tensor v, torch::Tensor gate) {
-  TORCH_CHECK(v.is_cuda() && v.dim() == 3 && v.stride(2) == 1);
-  const int H = v.size(0), T = v.size(1), VD = v.size(2);
-  TORCH_CHECK(out.is_contiguous() && out.dtype() == v.dtype() &&
-              out.numel() == (int64_t)H * T * VD);
-  TORCH_CHECK(gate.is_contiguous() && gate.dtype() == torch::kFloat32 &&
-              gate.size(0) == T && gate.size(1) == H);
-  const int64_t total = (int64_t)H * T * VD;
-  if (total == 0) return;
-  hipStream_t stream = at::cuda::getCurrentCUDAStream();
-  IGW_DISPATCH_ACT(v, {
-    hipLaunchKernelGGL((gate_heads_kernel<act_t>), dim3((total + 255) / 256),
-                       dim3(256), 0, stream, (act_t*)out.data_ptr(),
-                       (const act_t*)v.data_ptr(), (int64_t)v.stride(0),
-                       (int64_t)v.stride(1), (const float*)gate.data_ptr(), H,
-                       VD, total);
   });
   HIP_CHECK_KERNEL();
 }

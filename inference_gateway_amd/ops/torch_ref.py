@@ -462,13 +462,6 @@ def relu2_ref(z):
     return (r * r).to(z.dtype)
 
 
-def gate_heads_ref(v, gate):
-    """v [H, T, vd] per-head values, gate [T, H] fp32 -> [T, H*vd]."""
-    H, T, vd = v.shape
-    return (v.float().transpose(0, 1) * gate[:, :, None]).reshape(
-        T, H * vd).to(v.dtype)
-
-
 def moe_topk_route_ref(logits, top_k):
     """Top-k experts by logit and the softmax over just those k."""
     w, idx = torch.topk(logits, top_k, dim=-1)
