@@ -74,12 +74,14 @@ class LatentAttentionSpec:
     rot_dim: int = 16          # rotated q/k entries per head (shared key)
     vdim: int = 64             # value entries per head
     kv_rank: int = 64          # cached latent width
-    q_rank: int = 64           # query latent width
+    q_rank: int = 64           # query latent width; 0 = queries are
+                               #   projected straight from the input
     scale: float = 0.0         # score multiplier; 0 => (dim+rot_dim)**-0.5
     window: int = 0            # keys seen per query incl. itself; 0 = all
     rot: object = None         # RotarySpec | YarnRotarySpec
     rot_half: bool = False     # pairs (i, i + dims/2) instead of (2i, 2i+1)
     sink: bool = True          # learned softmax sink per head
+    gate: bool = True          # sigmoid output gate per head
     kv_from: int = -1          # layer whose cached rows are read (-1 = own)
 
     def __post_init__(self):
@@ -689,19 +691,28 @@ class ChunkBiasAttentionSpec:
 
 @dataclass
 class SinkAttentionSpec:
-    """Causal softmax attention with projection biases, per-head RMS
-    norm of queries and keys, partial rotary positions, and one more
-    term of score 0 and no value in the softmax denominator."""
+    """Causal softmax attention with projection biases, optional
+    per-head RMS norm of queries and keys, partial rotary positions, and
+    one more term without a value in the softmax denominator, of score 0
+    or of one learned score per head.  With tied_values the value of a
+    token is its projected key before norm and rotation."""
     heads: int = 1
     kv_heads: int = 1
     dim: int = 64
     vdim: int = 64
     scale: float = 0.0         # 0 => dim ** -0.5
     rot: YarnRotarySpec = None  # None => no rotation
+    rot_half: bool = False     # pairs (i, i + dims/2) instead of (2i, 2i+1)
+    qk_norm: bool = True
+    learned_sink: bool = False
+    tied_values: bool = False
+    out_bias: bool = False
 
     def __post_init__(self):
         if not self.scale:
             self.scale = float(self.dim) ** -0.5
+        if self.tied_values and self.vdim != self.dim:
+            raise ValueError("values tied to the keys have the keys' width")
 
 
 @dataclass
@@ -1069,6 +1080,225 @@ def bivatar_preset(name: str, width: int, vocab: int, pattern: str,
                          residual_mult=residual_mult)
 
 
+# ---------------------------------------------------------------------------
+# Defosun: a per-layer decoder with several residual streams in place of
+# one residual sum, and a run of neighbouring layers that repeats with the
+# same weights.  Mixers: softmax attention whose values are its unrotated
+# keys, with learned sinks; latent attention with direct queries and
+# sinks; linear attention with a fixed decay per head.  Feed-forward:
+# silu-gated dense unit, or clamped experts behind a softmax router plus a
+# gated shared expert, or none.
+# ---------------------------------------------------------------------------
+@dataclass
+class FixedDecaySpec:
+    """Linear attention: S <- decay_h S + k v^T, o = S^T q per head, with
+    silu on q, k and v; the concatenated heads RMS-normed together, times
+    a sigmoid gate."""
+    heads: int = 1
+    dim: int = 64
+    vdim: int = 64
+    decay: tuple = (1.0,)      # one factor per head
+
+    def __post_init__(self):
+        self.decay = tuple(float(d) for d in self.decay)
+        if len(self.decay) != self.heads:
+            raise ValueError(f"{len(self.decay)} decays for {self.heads} "
+                             "heads")
+
+
+@dataclass
+class SiluFFSpec:
+    """W_down (silu(W_gate h) * (W_up h))."""
+    ff: int = 0
+
+
+@dataclass
+class SharedClampedMoESpec:
+    """Clamped gated experts chosen by the largest entries of a softmax
+    over all router logits and weighted by those entries as they are,
+    beside an optional shared expert of the same form behind one sigmoid
+    gate per token."""
+    experts: int = 1
+    top: int = 1
+    expert_ff: int = 0
+    limit: float = 7.0
+    shared_ff: int = 0         # 0 => no shared expert
+    shared_limit: float = 7.0
+
+
+@dataclass
+class DefosunConfig:
+    name: str
+    hidden_size: int
+    vocab_size: int
+    layers: list        # LayerSpec(type="attention"|"latent_attention"|
+                        #           "lightning")
+    norm_eps: float = 1e-6
+    streams: int = 1
+    loop_start: int = 0        # layers loop_start .. loop_stop - 1 run
+    loop_stop: int = 0         # loop_times times in a row
+    loop_times: int = 1
+    max_position: int = 1 << 20     # angles are computed, not tabulated
+    architecture: str = "Defosun"
+
+    def __post_init__(self):
+        if self.streams < 1:
+            raise ValueError("at least one residual stream")
+        if self.loop_stop == self.loop_start:
+            self.loop_times = 1
+        if not (0 <= self.loop_start <= self.loop_stop <= len(self.layers)
+                and self.loop_times >= 1):
+            raise ValueError(
+                f"loop {self.loop_start} .. {self.loop_stop} x "
+                f"{self.loop_times} does not fit {len(self.layers)} layers")
+
+    @property
+    def num_layers(self) -> int:
+        return len(self.layers)
+
+    @property
+    def layer_runs(self) -> list:
+        """Layer numbers in the order they run."""
+        a, b = self.loop_start, self.loop_stop
+        return (list(range(a)) + list(range(a, b)) * self.loop_times
+                + list(range(b, len(self.layers))))
+
+    @property
+    def is_moe(self) -> bool:
+        return any(isinstance(l.mlp, SharedClampedMoESpec)
+                   for l in self.layers)
+
+    def kv_bytes_per_token(self, itemsize: int = 2) -> int:
+        """Paged bytes per token: keys and values, and latent rows, of
+        every layer RUN (a repeated layer has a cache per pass)."""
+        n = 0
+        for i in self.layer_runs:
+            l, m = self.layers[i], self.layers[i].mixer
+            if l.type == "attention":
+                n += m.kv_heads * (m.dim + m.vdim) * itemsize
+            elif l.type == "latent_attention":
+                n += m.cache_width * itemsize
+        return max(itemsize, n)
+
+    @staticmethod
+    def from_dict(cfg: dict, name: str = "defosun",
+                  shapes: Optional[dict] = None) -> "DefosunConfig":
+        """Parse the design's config.json.  `shapes` (tensor name ->
+        shape, from the checkpoint header) fills sizes that the json
+        leaves to the tensors."""
+        shapes = shapes or {}
+
+        def size(entry, key, tensor, axis=0):
+            v = (entry or {}).get(key)
+            return int(shapes[tensor][axis] if v is None else v)
+
+        layers = []
+        for i, l in enumerate(cfg["layers"]):
+            m = l.get("mixer") or {}
+            t = l["type"]
+            if t == "attention":
+                dim = int(m["dim"])
+                mixer = SinkAttentionSpec(
+                    heads=int(m["heads"]),
+                    kv_heads=int(m.get("kv_heads") or m["heads"]),
+                    dim=dim, vdim=int(m.get("vdim") or dim),
+                    scale=float(m.get("scale") or 0.0),
+                    rot=YarnRotarySpec.from_dict(m.get("rot")),
+                    rot_half=True, qk_norm=False, learned_sink=True,
+                    tied_values=True, out_bias=True)
+            elif t == "latent_attention":
+                rot = YarnRotarySpec.from_dict(m.get("rot"))
+                rd = m.get("rot_dim")
+                mixer = LatentAttentionSpec(
+                    heads=int(m["heads"]), dim=int(m["dim"]),
+                    rot_dim=int(rot.dims if rd is None else rd),
+                    vdim=int(m.get("vdim") or m["dim"]),
+                    kv_rank=size(m, "kv_rank", f"l{i}.mix.dkv.norm"),
+                    q_rank=0, scale=float(m.get("scale") or 0.0), rot=rot,
+                    sink=True, gate=False)
+            elif t == "lightning":
+                mixer = FixedDecaySpec(
+                    heads=int(m["heads"]), dim=int(m["dim"]),
+                    vdim=int(m.get("vdim") or m["dim"]),
+                    decay=tuple(m["decay"]))
+            else:
+                raise ValueError(f"layer {i}: unknown mixer {t!r}")
+            f, p = l.get("mlp"), f"l{i}.mlp."
+            if f is None:
+                mlp = None
+            elif f["kind"] == "dense":
+                mlp = SiluFFSpec(ff=size(f, "ff", p + "gate"))
+            elif f["kind"] == "moe":
+                ex, sh, r = f.get("expert") or {}, f.get("shared"), \
+                    f.get("router") or {}
+                mlp = SharedClampedMoESpec(
+                    experts=size(r, "experts", p + "router"),
+                    top=int(r["top"]),
+                    expert_ff=size(ex, "ff", p + "e0.gate"),
+                    limit=float(ex["limit"]))
+                if sh is not None:
+                    mlp.shared_ff = size(sh, "ff", p + "shared.gate")
+                    mlp.shared_limit = float(sh["limit"])
+            else:
+                raise ValueError(f"layer {i}: unknown mlp {f['kind']!r}")
+            layers.append(LayerSpec(type=t, mixer=mixer, mlp=mlp))
+        loop = cfg.get("loop") or {}
+        return DefosunConfig(
+            name=name, hidden_size=int(cfg["width"]),
+            vocab_size=int(cfg["vocab"]), layers=layers,
+            norm_eps=float((cfg.get("norm") or {}).get("eps", 1e-6)),
+            streams=int(cfg.get("streams") or 1),
+            loop_start=int(loop.get("start") or 0),
+            loop_stop=int(loop.get("stop") or 0),
+            loop_times=int(loop.get("times", 1)))
+
+
+def defosun_preset(name: str, width: int, vocab: int, pattern: str,
+                   heads: int, kv_heads: int, dim: int, rot_dims: int,
+                   l_dim: int, rot_dim: int, l_vdim: int, kv_rank: int,
+                   d_dim: int, d_vdim: int, ff: int, experts: int, top: int,
+                   expert_ff: int, shared_ff: int = 0, streams: int = 4,
+                   loop: tuple = (0, 0, 1), limit: float = 7.0,
+                   rot_base: float = 10000.0, l_heads: int = 0,
+                   d_heads: int = 0) -> DefosunConfig:
+    """Layer pattern string: two letters per layer — mixer `a`
+    (attention), `l` (latent attention) or `f` (fixed-decay linear
+    attention), then `d` (dense), `m` (experts) or `-` (no
+    feed-forward); e.g. "ad fm ad lm".  loop = (start, stop, times)."""
+    dh = d_heads or heads
+    layers = []
+    for mx, f in pattern.split():
+        if mx == "a":
+            typ, mixer = "attention", SinkAttentionSpec(
+                heads=heads, kv_heads=kv_heads, dim=dim, vdim=dim,
+                rot=YarnRotarySpec(base=rot_base, dims=rot_dims),
+                rot_half=True, qk_norm=False, learned_sink=True,
+                tied_values=True, out_bias=True)
+        elif mx == "l":
+            typ, mixer = "latent_attention", LatentAttentionSpec(
+                heads=l_heads or heads, dim=l_dim, rot_dim=rot_dim,
+                vdim=l_vdim, kv_rank=kv_rank, q_rank=0,
+                rot=YarnRotarySpec(base=rot_base, dims=rot_dim),
+                sink=True, gate=False)
+        else:
+            typ, mixer = "lightning", FixedDecaySpec(
+                heads=dh, dim=d_dim, vdim=d_vdim,
+                decay=tuple(1.0 - 2.0 ** (-1.0 - 9.0 * h / max(1, dh - 1))
+                            for h in range(dh)))
+        mlp = None
+        if f == "d":
+            mlp = SiluFFSpec(ff=ff)
+        elif f == "m":
+            mlp = SharedClampedMoESpec(
+                experts=experts, top=top, expert_ff=expert_ff, limit=limit,
+                shared_ff=shared_ff, shared_limit=limit)
+        layers.append(LayerSpec(type=typ, mixer=mixer, mlp=mlp))
+    return DefosunConfig(
+        name=name, hidden_size=width, vocab_size=vocab, layers=layers,
+        norm_eps=1e-5, streams=streams, loop_start=loop[0],
+        loop_stop=loop[1], loop_times=loop[2])
+
+
 # Architectures from the public model cards (random-init weights — no network).
 MODEL_PRESETS = {
     "llama-3-8b": ModelConfig(
@@ -1255,6 +1485,20 @@ MODEL_PRESETS = {
         heads=32, kv_heads=8, dim=128, vdim=128, window=1024,
         keep_first=16, l_dim=128, rot_dim=64, l_vdim=128, kv_rank=512,
         q_rank=1536, ff=14336, yarn_factor=8.0, yarn_original=4096.0),
+    # tiny Defosun for CPU tests / smoke: the three mixers, both
+    # feed-forwards, a layer without one, two layers that run twice
+    "tiny-defosun": defosun_preset(
+        "tiny-defosun", width=96, vocab=320, pattern="ad fm lm a-",
+        heads=4, kv_heads=2, dim=24, rot_dims=16, l_dim=16, rot_dim=8,
+        l_vdim=24, kv_rank=40, d_dim=16, d_vdim=24, ff=160, experts=6,
+        top=2, expert_ff=40, shared_ff=56, streams=3, loop=(1, 3, 2),
+        limit=1.5),
+    # layer-shape benchmark point at Llama-3-8B's width
+    "defosun-4k": defosun_preset(
+        "defosun-4k", width=4096, vocab=32000, pattern="ad fm ad lm",
+        heads=32, kv_heads=8, dim=128, rot_dims=64, l_dim=128, rot_dim=64,
+        l_vdim=128, kv_rank=512, d_dim=128, d_vdim=128, ff=14336,
+        experts=8, top=2, expert_ff=7168, shared_ff=7168),
     "tiny-moe": ModelConfig(
         name="tiny-moe",
         hidden_size=512,
@@ -1421,6 +1665,19 @@ class EngineConfig:
     def tiny_bivatar(**kw) -> "EngineConfig":
         defaults = dict(
             model=MODEL_PRESETS["tiny-bivatar"],
+            num_gpu_blocks=64,
+            max_num_seqs=8,
+            max_batched_tokens=2048,
+            max_model_len=512,
+            use_hip_graphs=False,
+        )
+        defaults.update(kw)
+        return EngineConfig(**defaults)
+
+    @staticmethod
+    def tiny_defosun(**kw) -> "EngineConfig":
+        defaults = dict(
+            model=MODEL_PRESETS["tiny-defosun"],
             num_gpu_blocks=64,
             max_num_seqs=8,
             max_batched_tokens=2048,

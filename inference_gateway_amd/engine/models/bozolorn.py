@@ -106,22 +106,29 @@ class ChunkBiasAttention(nn.Module):
 
 
 class SinkRotaryAttention(nn.Module):
-    """q, k, v = W h + b; q and k RMS-normed per head (one weight vector
-    shared by the heads) and rotated on their first rot.dims entries;
-    causal; p_j = exp(s_j) / (1 + sum exp(s)); W_o."""
+    """q, k, v = W h + b; q and k rotated on their first rot.dims entries
+    (either pair layout); causal; p_j = exp(s_j) / (exp(sink_h) + sum
+    exp(s)); W_o (+ b).  By the spec: q and k RMS-normed per head first
+    (one weight vector shared by the heads) or not; sinks learned per head
+    or 0; values projected or the keys as projected."""
 
     def __init__(self, hidden: int, spec: SinkAttentionSpec, eps: float,
                  name: str, device, dtype):
         super().__init__()
         self.spec, self.eps = spec, eps
         H, G, N, P = spec.heads, spec.kv_heads, spec.dim, spec.vdim
-        rows = H * N + G * N + G * P
+        # fused projection rows: q | k | v (own values only)
+        rows = H * N + G * N + (0 if spec.tied_values else G * P)
         self.qkv = _w((rows, hidden), device, dtype, name + ".qkv", hidden)
         self.qkv_b = _param(_rand((rows,), device, dtype, name + ".qkv_b",
                                   10.0))
-        self.qnorm_w = _norm_w(N, device, name + ".q.norm")
-        self.knorm_w = _norm_w(N, device, name + ".k.norm")
+        self.qnorm_w = self.knorm_w = None
+        if spec.qk_norm:
+            self.qnorm_w = _norm_w(N, device, name + ".q.norm")
+            self.knorm_w = _norm_w(N, device, name + ".k.norm")
         self.o = _w((hidden, H * P), device, dtype, name + ".o", H * P)
+        self.o_b = _param(_rand((hidden,), device, dtype, name + ".o_b",
+                                10.0)) if spec.out_bias else None
         self.mag = 1.0
         if spec.rot is not None and spec.rot.dims > 0:
             freq, self.mag = spec.rot.frequencies()
@@ -130,9 +137,13 @@ class SinkRotaryAttention(nn.Module):
                 persistent=False)
         else:
             self.inv_freq = None
-        # the sink: one more softmax term of score 0 for every head
-        self.register_buffer("sinks", torch.zeros(
-            H, dtype=torch.float32, device=device), persistent=False)
+        if spec.learned_sink:
+            self.sinks = _param(_rand((H,), device, torch.float32,
+                                      name + ".sink", 25.0))
+        else:
+            # one more softmax term of score 0 for every head
+            self.register_buffer("sinks", torch.zeros(
+                H, dtype=torch.float32, device=device), persistent=False)
 
     def cache_spec(self):
         s = self.spec
@@ -145,12 +156,12 @@ class SinkRotaryAttention(nn.Module):
         q = ops.qk_norm_rope_append(
             proj, fb.positions, fb.slot_mapping, kc, vc, self.qnorm_w,
             self.knorm_w, self.inv_freq, self.mag, self.eps, s.heads,
-            s.kv_heads, s.dim, s.vdim)
+            s.kv_heads, s.dim, s.vdim, s.rot_half, s.tied_values)
         o = ops.softcap_attention(
             q, kc, vc, fb.seq_block_table, fb.row_seq, fb.positions,
             s.scale, 0.0, 0.0, 1, 0, fb.num_chunk_rows, fb.seq_lens,
             fb.seq_cu, fb.seq_start, sinks=self.sinks)
-        return F.linear(o, self.o)
+        return F.linear(o, self.o, self.o_b)
 
 
 class GatedDeltaMixer(nn.Module):

@@ -98,9 +98,11 @@ class LatentAttention(nn.Module):
     after the probability-weighted sum of latents, so every head reads
     the same cached row (latent | rotated key) — prefill portions and
     decoded tokens both attend straight out of the paged cache.  The
-    per-head output gate is applied to the latent sum (it commutes with
-    the value up-projection).  A layer with spec.kv_from >= 0 has no
-    key/value projection and reads the rows of that layer."""
+    per-head output gate (spec.gate) is applied to the latent sum (it
+    commutes with the value up-projection).  With spec.q_rank 0 the
+    queries are projected straight from the input, in the same GEMM as the
+    latent.  A layer with spec.kv_from >= 0 has no key/value projection
+    and reads the rows of that layer."""
 
     cache_kind = "latent"
 
@@ -113,18 +115,25 @@ class LatentAttention(nn.Module):
         R, vd, qr = spec.kv_rank, spec.vdim, spec.q_rank
         s = hidden ** -0.5 / 0.02
         self.owns_kv = spec.kv_from < 0
-        # fused down projection: query latent | kv latent | rotated key
-        # (own keys only) | per-head output-gate logits
-        rows = qr + (R + rd if self.owns_kv else 0) + H
+        self.direct = qr == 0
+        if self.direct and (spec.gate or not self.owns_kv):
+            raise ValueError("direct queries go with own keys and no gate")
+        if not self.direct and not spec.gate:
+            raise ValueError("a query latent goes with an output gate")
+        # fused down projection: query latent (direct: queries) | kv latent
+        # | rotated key (own keys only) | per-head output-gate logits
+        rows = (R + rd if self.owns_kv else 0) + (
+            H * (dn + rd) if self.direct else qr + H)
         self.down = _param(_rand((rows, hidden), device, dtype,
                                  name + ".down", s))
-        self.qnorm_w = _param(1.0 + _rand((qr,), device, torch.float32,
-                                          name + ".qn", 2.0))
+        self.qnorm_w = None if self.direct else _param(
+            1.0 + _rand((qr,), device, torch.float32, name + ".qn", 2.0))
         self.kvnorm_w = _param(1.0 + _rand(
             (R,), device, torch.float32, name + ".kvn", 2.0)) \
             if self.owns_kv else None
-        self.uq = _param(_rand((H * (dn + rd), qr), device, dtype,
-                               name + ".uq", qr ** -0.5 / 0.02))
+        self.uq = None if self.direct else _param(
+            _rand((H * (dn + rd), qr), device, dtype, name + ".uq",
+                  qr ** -0.5 / 0.02))
         # absorbed forms, per head: uk [H, dn, R] maps an unrotated query
         # to latent space; uv_t [H, R, vd] maps a latent sum to values
         self.uk = _param(_rand((H, dn, R), device, dtype, name + ".uk",
@@ -154,14 +163,22 @@ class LatentAttention(nn.Module):
         T = h.shape[0]
         H, dn, rd = sp.heads, sp.dim, sp.rot_dim
         down = F.linear(h, self.down)
-        cq, gate = ops.latent_down_post(
-            down, fb.positions, fb.slot_mapping,
-            cache if self.owns_kv else None, self.qnorm_w, self.kvnorm_w,
-            self.inv_freq, self.eps, sp.q_rank, sp.kv_rank, rd, H,
-            sp.rot_half, self.mag)
-        q = F.linear(cq, self.uq).view(T, H, dn + rd)
-        ops.rope_pairs_(q, fb.positions, self.inv_freq, dn, sp.rot_half,
-                        self.mag)
+        if self.direct:
+            gate = None
+            ops.latent_rope_append(
+                down, fb.positions, fb.slot_mapping, cache, self.kvnorm_w,
+                self.inv_freq, self.eps, H, dn, rd, sp.kv_rank, sp.rot_half,
+                self.mag)
+            q = down[:, :H * (dn + rd)].view(T, H, dn + rd)
+        else:
+            cq, gate = ops.latent_down_post(
+                down, fb.positions, fb.slot_mapping,
+                cache if self.owns_kv else None, self.qnorm_w,
+                self.kvnorm_w, self.inv_freq, self.eps, sp.q_rank,
+                sp.kv_rank, rd, H, sp.rot_half, self.mag)
+            q = F.linear(cq, self.uq).view(T, H, dn + rd)
+            ops.rope_pairs_(q, fb.positions, self.inv_freq, dn, sp.rot_half,
+                            self.mag)
         q_abs = torch.bmm(q[:, :, :dn].transpose(0, 1), self.uk)  # [H,T,R]
         o_lat = ops.latent_attention(
             q_abs.transpose(0, 1), q[:, :, dn:], cache, fb.seq_block_table,

@@ -85,3 +85,40 @@ def padded_rows(topk_idx: torch.Tensor, num_experts: int, capacity: int
     oh = torch.nn.functional.one_hot(flat_e, num_experts)
     rank = (torch.cumsum(oh, 0) - oh).mul(oh).sum(-1)
     return flat_e * capacity + rank
+
+
+def experts_combined(x: torch.Tensor, weights: torch.Tensor,
+                     topk_idx: torch.Tensor, dst, capacity: int,
+                     up_t: torch.Tensor, down_t: torch.Tensor,
+                     act: Callable[[torch.Tensor], torch.Tensor],
+                     shared=None, shared_gate=None) -> torch.Tensor:
+    """Either route with the dispatch and the weighted sum as one kernel
+    each (ops.moe_scatter_rows, ops.moe_combine), the sum taking an
+    optional shared expert's rows times sigmoid(shared_gate [T] fp32).
+    dst: padded rows for the padded route (capacity rows per expert);
+    None takes the sorted route, one gather and one contiguous GEMM pair
+    per non-empty expert."""
+    from ... import ops
+
+    T, h = x.shape
+    E, K = up_t.shape[0], weights.shape[1]
+    if dst is not None:
+        buf = ops.moe_scatter_rows(x, dst, E * capacity)
+        mid = torch.bmm(buf.view(E, capacity, h), up_t)
+        a = act(mid.view(E * capacity, -1))
+        y = torch.bmm(a.view(E, capacity, -1), down_t).view(E * capacity, h)
+    else:
+        flat_e = topk_idx.reshape(-1).long()
+        order = torch.argsort(flat_e, stable=True)
+        counts = torch.bincount(flat_e, minlength=E).tolist()
+        xs = x.index_select(0, torch.div(order, K, rounding_mode="floor"))
+        y = torch.empty((T * K, h), dtype=x.dtype, device=x.device)
+        at = 0
+        for e, n in enumerate(counts):
+            if n:
+                torch.mm(act(torch.mm(xs[at:at + n], up_t[e])), down_t[e],
+                         out=y[at:at + n])
+            at += n
+        dst = torch.empty_like(order)
+        dst[order] = torch.arange(T * K, device=x.device)
+    return ops.moe_combine(y, dst, weights, shared, shared_gate)

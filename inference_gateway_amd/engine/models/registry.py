@@ -8,8 +8,9 @@ from pathlib import Path
 
 import torch
 
-from ..config import (BivatarConfig, BozolornConfig, FedatarConfig,
-                      FeditarConfig, MekevikConfig, ModelConfig)
+from ..config import (BivatarConfig, BozolornConfig, DefosunConfig,
+                      FedatarConfig, FeditarConfig, MekevikConfig,
+                      ModelConfig)
 
 
 def build_model(model_cfg, device, dtype):
@@ -24,6 +25,8 @@ def build_model(model_cfg, device, dtype):
         from .bozolorn import BozolornForCausalLM as cls
     elif isinstance(model_cfg, BivatarConfig):
         from .bivatar import BivatarForCausalLM as cls
+    elif isinstance(model_cfg, DefosunConfig):
+        from .defosun import DefosunForCausalLM as cls
     elif model_cfg.is_moe:
         from .mixtral import MixtralForCausalLM as cls
     else:
@@ -72,6 +75,10 @@ def model_config_from_dir(path: str):
         return BivatarConfig.from_dict(
             cfg, name=Path(path).name or "bivatar",
             shapes=safetensors_shapes(path))
+    if cfg.get("architecture") == "Defosun":
+        return DefosunConfig.from_dict(
+            cfg, name=Path(path).name or "defosun",
+            shapes=safetensors_shapes(path))
     if cfg.get("architecture") == "Fedatar":
         return FedatarConfig.from_dict(
             cfg, name=Path(path).name or "fedatar",
@@ -90,10 +97,13 @@ def is_recurrent(model_cfg) -> bool:
     if isinstance(model_cfg, BozolornConfig):
         # the delta-rule half of a parallel mixer keeps slot state
         return any(l.type == "parallel" for l in model_cfg.layers)
+    if isinstance(model_cfg, DefosunConfig):
+        return any(l.type == "lightning" for l in model_cfg.layers)
     return isinstance(model_cfg, FedatarConfig) and any(
         l.type == "mingru" for l in model_cfg.layers)
 
 
 __all__ = ["build_model", "model_config_from_dir", "safetensors_shapes",
            "is_recurrent", "ModelConfig", "FedatarConfig", "MekevikConfig",
-           "FeditarConfig", "BozolornConfig", "BivatarConfig"]
+           "FeditarConfig", "BozolornConfig", "BivatarConfig",
+           "DefosunConfig"]

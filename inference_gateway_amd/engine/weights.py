@@ -613,6 +613,88 @@ def load_bivatar_weights(model, path: str) -> int:
     return n
 
 
+def load_defosun_weights(model, path: str) -> int:
+    """Load a Defosun checkpoint: tensors `embed`, `l<i>.norm1|norm2`,
+    `l<i>.hc1|hc2.{in,out,mix}`, `l<i>.mix.*` per mixer kind,
+    `l<i>.mlp.{gate,up,down}` or `l<i>.mlp.router`,
+    `l<i>.mlp.e<j>.{gate,up,down}` and `l<i>.mlp.shared.{gate,up,down,sg}`,
+    `final.norm`, `head`.  The engine's layouts are assembled here: q|k
+    with their biases stacked for the attention input GEMM, q|dkv for the
+    latent attention's (up-projections per head in absorbed form), q|k|v|g
+    for the fixed-decay attention's; router and shared gate stacked in
+    fp32; experts stacked K-major with gate|up side by side.  Norm weights
+    stored around zero are held as 1 + w in fp32."""
+    sh = _Shards(path)
+    cfg = model.cfg
+    n = 0
+
+    def put(param, src, what):
+        nonlocal n
+        _copy(param, src, what)
+        n += 1
+
+    def cat(prefix, names, suffix=""):
+        return torch.cat([sh.full(prefix + c + suffix) for c in names], 0)
+
+    def put_norm(param, what):
+        put(param, 1.0 + sh.full(what).float(), what)
+
+    def put_streams(hc, prefix):
+        put(hc.inw, sh.full(prefix + "in"), prefix + "in")
+        put(hc.outw, sh.full(prefix + "out"), prefix + "out")
+        put(hc.mix, sh.full(prefix + "mix"), prefix + "mix")
+
+    put(model.embed, sh.full("embed"), "embed")
+    for i, (spec, layer) in enumerate(zip(cfg.layers, model.layers)):
+        p = f"l{i}."
+        put_norm(layer.norm1_w, p + "norm1")
+        put_streams(layer.hc1, p + "hc1.")
+        mx, m, a = layer.mixer, p + "mix.", spec.mixer
+        if spec.type == "attention":
+            put(mx.qkv, cat(m, "qk"), m + "q|k")
+            put(mx.qkv_b, cat(m, "qk", ".b"), m + "q|k.b")
+            put(mx.sinks, sh.full(m + "sink"), m + "sink")
+            put(mx.o_b, sh.full(m + "o.b"), m + "o.b")
+        elif spec.type == "latent_attention":
+            put(mx.down, cat(m, ("q", "dkv")), m + "q|dkv")
+            put(mx.kvnorm_w, sh.full(m + "dkv.norm"), m + "dkv.norm")
+            put(mx.uk, sh.full(m + "uk").view(a.heads, a.dim, a.kv_rank),
+                m + "uk")
+            put(mx.uv_t, sh.full(m + "uv").view(
+                a.heads, a.vdim, a.kv_rank).transpose(1, 2), m + "uv")
+            put(mx.sink, sh.full(m + "sink"), m + "sink")
+        else:
+            put(mx.qkvg, cat(m, "qkvg"), m + "q|k|v|g")
+            put(mx.norm_w, sh.full(m + "norm"), m + "norm")
+        put(mx.o, sh.full(m + "o"), m + "o")
+        if spec.mlp is None:
+            continue
+        put_norm(layer.norm2_w, p + "norm2")
+        put_streams(layer.hc2, p + "hc2.")
+        f, ff = layer.mlp, p + "mlp."
+        if not hasattr(f, "router_w"):
+            put(f.gate_up, cat(ff, ("gate", "up")), ff + "gate|up")
+            put(f.down, sh.full(ff + "down"), ff + "down")
+            continue
+        has_shared = f.shared_up is not None
+        rows = ("router", "shared.sg") if has_shared else ("router",)
+        put(f.router_w, cat(ff, rows), ff + "|".join(rows))
+        E = spec.mlp.experts
+        put(f.up_t, torch.stack([cat(ff + f"e{e}.", ("gate", "up")).t()
+                                 for e in range(E)]), ff + "e*.gate|up")
+        put(f.down_t, torch.stack(
+            [sh.full(ff + f"e{e}.down").t() for e in range(E)]),
+            ff + "e*.down")
+        if has_shared:
+            put(f.shared_up, cat(ff + "shared.", ("gate", "up")),
+                ff + "shared.gate|up")
+            put(f.shared_down, sh.full(ff + "shared.down"),
+                ff + "shared.down")
+    put_norm(model.final_norm_w, "final.norm")
+    put(model.head, sh.full("head"), "head")
+    return n
+
+
 def _is_gguf(path: str) -> bool:
     p = Path(path)
     if p.is_file():
@@ -642,6 +724,8 @@ def load_weights(model, path: str) -> int:
         return load_bozolorn_weights(model, path)
     if getattr(model.cfg, "architecture", "") == "Bivatar":
         return load_bivatar_weights(model, path)
+    if getattr(model.cfg, "architecture", "") == "Defosun":
+        return load_defosun_weights(model, path)
     if getattr(model.cfg, "is_moe", False):
         return load_mixtral_weights(model, path)
     return load_llama_weights(model, path)

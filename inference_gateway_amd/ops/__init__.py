@@ -49,6 +49,15 @@ except ImportError:  # pragma: no cover - absent only before first build
     HAS_POSTNORM = False
 
 
+try:
+    from . import _streams  # residual streams, fixed-decay attention
+
+    HAS_STREAMS = True
+except ImportError:  # pragma: no cover - absent only before first build
+    _streams = None
+    HAS_STREAMS = False
+
+
 def _require_recurrent() -> None:
     if not HAS_RECURRENT:
         raise RuntimeError(
@@ -59,11 +68,19 @@ def _require_recurrent() -> None:
         )
 
 
+def _require_streams() -> None:
+    if not HAS_STREAMS:
+        raise RuntimeError(
+            "inference_gateway_amd.ops._streams is not built but a GPU "
+            "tensor was passed. Build it in-tree with: IGW_BUILD_EXT=streams "
+            "PYTORCH_ROCM_ARCH=gfx950 python setup.py build_ext --inplace")
+
+
 def _shared_ext(name: str):
     """An op that several extensions compile (same source file):
     whichever is built serves it, so a process that runs one model family
     needs one library."""
-    for ext in (_postnorm, _hybrid, _recurrent):
+    for ext in (_postnorm, _streams, _hybrid, _recurrent):
         if ext is not None and hasattr(ext, name):
             return getattr(ext, name)
     raise RuntimeError(
@@ -476,15 +493,15 @@ def relu2(z):
 
 
 def moe_topk_route(logits, top_k: int, capacity: int = 0,
-                   scale: float = 1.0):
-    """logits [T, E] fp32 -> (softmax-over-chosen weights [T, K] fp32
-    times `scale`,
+                   scale: float = 1.0, over_all: bool = False):
+    """logits [T, E] fp32 (strided rows ok) -> (weights [T, K] fp32 =
+    softmax over the chosen logits, or with over_all the chosen entries of
+    the softmax over all E, times `scale`,
     expert ids [T, K] int32, padded rows [T*K] int64 or None).  With
     capacity > 0 (>= T) the padded-dispatch row of every assignment,
     expert * capacity + rank, comes from the same launch.  Any K <= E <=
     64 on the GPU kernel, wider routers take the library top-k."""
     if logits.is_cuda and logits.shape[1] <= 64:
-        _require_hybrid()
         T, E = logits.shape
         w = torch.empty((T, top_k), dtype=torch.float32,
                         device=logits.device)
@@ -495,10 +512,10 @@ def moe_topk_route(logits, top_k: int, capacity: int = 0,
             dst = torch.empty(T * top_k, dtype=torch.int64,
                               device=logits.device)
             counts = torch.zeros(E, dtype=torch.int32, device=logits.device)
-        _hybrid.moe_topk_route(w, idx, logits, dst, counts, capacity,
-                               scale)
+        _shared_ext("moe_topk_route")(w, idx, logits, dst, counts, capacity,
+                                      scale, over_all)
         return w, idx, dst
-    w, idx = torch_ref.moe_topk_route_ref(logits, top_k)
+    w, idx = torch_ref.moe_topk_route_ref(logits, top_k, over_all)
     return (w * scale if scale != 1.0 else w), idx, None
 
 
@@ -745,11 +762,10 @@ def head_norm_gate(o, gate, w, eps: float, group: int, gate_act: int,
     (strided ok) applied before or after the norm.  Returns [T, C] in
     out_dtype."""
     if o.is_cuda:
-        _require_recurrent()
         T, H, P = o.shape
         out = torch.empty((T, H * P), dtype=out_dtype, device=o.device)
-        _recurrent.head_norm_gate(out, o, gate, w, eps, group, gate_act,
-                                  gate_first, den, floor)
+        _shared_ext("head_norm_gate")(out, o, gate, w, eps, group, gate_act,
+                                      gate_first, den, floor)
         return out
     return recurrent_ref.head_norm_gate_ref(o, gate, w, eps, group, gate_act,
                                             gate_first, den, floor,
@@ -834,25 +850,29 @@ def softcap_attention(q, kcache, vcache, block_table, row_seq, positions,
 
 def qk_norm_rope_append(proj, positions, slot_mapping, kcache, vcache,
                         qnorm_w, knorm_w, inv_freq, mag: float, eps: float,
-                        heads: int, kv_heads: int, dim: int, vdim: int):
+                        heads: int, kv_heads: int, dim: int, vdim: int,
+                        half: bool = False, tied: bool = False):
     """Post-processing of a fused projection [T, heads*dim | kv_heads*dim
     | kv_heads*vdim | ...] (strided rows ok): per-head RMS norm of the
     queries and keys (weights [dim] fp32 shared by the heads; None = no
-    norm), interleaved-pair rotation of each head's first
-    2*len(inv_freq) entries by position * inv_freq (fp32 angles, cos and
-    sin times `mag`; inv_freq None = no rotation), keys and values
-    appended to the paged caches [blocks, kv_heads, block, dim | vdim].
+    norm), pair rotation of each head's first 2*len(inv_freq) entries by
+    position * inv_freq (fp32 angles, cos and sin times `mag`; inv_freq
+    None = no rotation), keys and values appended to the paged caches
+    [blocks, kv_heads, block, dim | vdim].  Pairs are (2i, 2i+1), or with
+    `half` (i, i + len(inv_freq)).  `tied`: the projection has no value
+    block, a token's value is its projected key before norm and rotation.
     Returns the queries [T, heads*dim]."""
     if proj.is_cuda:
         q = torch.empty((proj.shape[0], heads * dim), dtype=proj.dtype,
                         device=proj.device)
         _shared_ext("qk_norm_rope_append")(
             q, proj, positions, slot_mapping, kcache, vcache, qnorm_w,
-            knorm_w, inv_freq, mag, eps, heads, kv_heads, dim, vdim)
+            knorm_w, inv_freq, mag, eps, heads, kv_heads, dim, vdim, half,
+            tied)
         return q
     return recurrent_ref.qk_norm_rope_append_ref(
         proj, positions, slot_mapping, kcache, vcache, qnorm_w, knorm_w,
-        inv_freq, mag, eps, heads, kv_heads, dim, vdim)
+        inv_freq, mag, eps, heads, kv_heads, dim, vdim, half, tied)
 
 
 def decay_beta_gates(pre, a_log, dt_bias):
@@ -958,3 +978,162 @@ def rmsnorm_pair_mean(a, b, wa, wb, eps: float):
         _recurrent.rmsnorm_pair_mean(out, a, b, wa, wb, eps)
         return out
     return recurrent_ref.rmsnorm_pair_mean_ref(a, b, wa, wb, eps)
+
+
+# ---------------------------------------------------------------------------
+# Multi-stream decoder mechanisms (extension _streams, CPU versions in
+# recurrent_ref): residual streams, fixed-decay linear attention, latent
+# attention input with direct queries, expert dispatch around a shared
+# expert.
+# ---------------------------------------------------------------------------
+def stream_step(streams, y, mix, outw, inw, norm_w, eps: float, out_dtype):
+    """Step between two sublayers of a model with B residual streams.
+    streams [T, B, D] fp32 (an expanded view is the same row in every
+    stream); y [T, D] = the previous sublayer's result or None.  With y,
+    the new streams are X'_t = sum_b mix[b, t] X_b + outw[t] y (mix [B, B]
+    indexed from, to); returns (streams, rmsnorm(sum_t inw[t] X'_t) *
+    norm_w in out_dtype).  Streams are updated in place where they can
+    be: use the returned ones.  All weights fp32."""
+    T, B, D = streams.shape
+    if streams.is_cuda:
+        _require_streams()
+        out = torch.empty((T, D), dtype=out_dtype, device=streams.device)
+        dst = None
+        if y is not None:
+            in_place = (streams.is_contiguous() and D % 4 == 0 and D <= 8192
+                        and B <= _streams.stream_step_max_in_place()
+                        and y.stride(0) % 4 == 0)
+            dst = streams if in_place else torch.empty(
+                (T, B, D), dtype=torch.float32, device=streams.device)
+        _streams.stream_step(out, streams, dst, y, mix, outw, inw, norm_w,
+                             eps)
+        return (streams if dst is None else dst), out
+    return recurrent_ref.stream_step_ref(streams, y, mix, outw, inw, norm_w,
+                                         eps, out_dtype)
+
+
+def latent_rope_append(x, positions, slot_mapping, cache, norm_w, inv_freq,
+                       eps: float, heads: int, dim: int, rot_dim: int,
+                       kv_rank: int, half: bool = False, mag: float = 1.0):
+    """x [T, heads*(dim+rot_dim) | kv_rank | rot_dim] (queries, latent,
+    shared key part): rotates the last rot_dim entries of every query head
+    in place and appends (RMS-normed latent | rotated shared key) to the
+    paged cache; half and mag as in rope_pairs_."""
+    if x.is_cuda:
+        _require_streams()
+        _streams.latent_rope_append(x, positions, slot_mapping, cache,
+                                    norm_w, inv_freq, eps, heads, dim,
+                                    rot_dim, kv_rank, half, mag)
+        return
+    recurrent_ref.latent_rope_append_ref(
+        x, positions, slot_mapping, cache, norm_w, inv_freq, eps, heads, dim,
+        rot_dim, kv_rank, half, mag)
+
+
+# sequences that bring at least this many rows run on the chunk kernel
+# (bf16, key width permitting); 0 = the step kernel for everything
+FIXED_DECAY_CHUNKS_FROM = 16
+FIXED_DECAY_CHUNK = 64
+# a launch of fewer workgroups than this cuts its sequences into segments
+FIXED_DECAY_MIN_BLOCKS = 256
+
+
+@functools.lru_cache(maxsize=256)
+def _decay_plan(seq_rows: tuple, blocks_per_segment: int, chunks: bool,
+                device):
+    """Who runs where: (sequences of the step kernel or None, segment
+    table [5, nseg] or None, segments per sequence as offsets or None =
+    one segment each).  Cached: serving repeats the same batch shapes."""
+    long = [i for i, n in enumerate(seq_rows)
+            if chunks and n >= FIXED_DECAY_CHUNKS_FROM > 0]
+    short = [i for i, n in enumerate(seq_rows) if n and i not in set(long)]
+    cu = [0]
+    for n in seq_rows:
+        cu.append(cu[-1] + n)
+
+    def dev(x):
+        return torch.tensor(x, dtype=torch.int32).to(device)
+
+    if not long:
+        return dev(short) if short else None, None, None
+    size = max(seq_rows[i] for i in long)
+    total = sum(seq_rows[i] for i in long)
+    if len(long) * blocks_per_segment < FIXED_DECAY_MIN_BLOCKS \
+            and size >= 4 * FIXED_DECAY_CHUNK:
+        want = -(-2 * FIXED_DECAY_MIN_BLOCKS // blocks_per_segment)
+        size = max(2 * FIXED_DECAY_CHUNK,
+                   -(-total // (want * FIXED_DECAY_CHUNK))
+                   * FIXED_DECAY_CHUNK)
+    tab, first = [], [0]
+    for i in long:
+        cuts = list(range(cu[i], cu[i + 1], size))
+        for a in cuts:
+            tab.append((a, min(a + size, cu[i + 1]), i, int(a == cuts[0]),
+                        int(a == cuts[-1])))
+        first.append(len(tab))
+    split = len(tab) > len(long)
+    return (dev(short) if short else None,
+            dev(list(zip(*tab))), dev(first) if split else None)
+
+
+def fixed_decay_scan(q, k, v, decay, state, seq_cu, seq_start, seq_slots,
+                     seq_rows, silu: bool = True):
+    """Linear attention with a fixed decay per head: S <- decay_h S + k_t
+    v_t^T, o_t = S^T q_t, S [N, P] fp32 in state [slots, H*N*P] (a
+    sequence whose first row is position 0 starts from zero).  q, k [T, G,
+    N] (strided ok; head h reads group h // (H/G)), v [T, H, P]; silu: all
+    three pass silu first.  decay [H] fp32.  Returns o fp32 [T, H, P].
+    seq_rows: python row counts per sequence."""
+    if v.is_cuda:
+        _require_streams()
+        T, H, P = v.shape
+        N = q.shape[2]
+        out = torch.empty((T, H, P), dtype=torch.float32, device=v.device)
+        chunks = (v.dtype == torch.bfloat16
+                  and N <= _streams.fixed_decay_chunk_keys())
+        per = H * (-(-P // 64) if P <= 64 else -(-P // 128))
+        short, segs, first = _decay_plan(tuple(seq_rows), per, chunks,
+                                         v.device)
+        if segs is not None:
+            work = None if first is None else torch.empty(
+                (segs.shape[1], H, N, P), dtype=torch.float32,
+                device=v.device)
+            _streams.fixed_decay_chunks(out, q, k, v, decay, state, segs,
+                                        work, first, seq_start, seq_slots,
+                                        silu)
+        if short is not None:
+            _streams.fixed_decay_step(out, q, k, v, decay, state, short,
+                                      seq_cu, seq_start, seq_slots, silu)
+        return out
+    return recurrent_ref.fixed_decay_scan_ref(q, k, v, decay, state, seq_cu,
+                                              seq_start, seq_slots, silu)
+
+
+def moe_scatter_rows(x, dst, rows: int):
+    """[rows, D] buffer with buf[dst[t*K + k]] = x[t] (dst int64 [T*K]);
+    rows that nothing is written to are left undefined."""
+    if x.is_cuda:
+        _require_streams()
+        buf = torch.empty((rows, x.shape[1]), dtype=x.dtype, device=x.device)
+        _streams.moe_scatter_rows(buf, x, dst, dst.numel() // x.shape[0])
+        return buf
+    buf = x.new_zeros((rows, x.shape[1]))
+    buf[dst] = x.repeat_interleave(dst.numel() // x.shape[0], 0)
+    return buf
+
+
+def moe_combine(y, dst, weights, shared=None, shared_gate=None):
+    """out [T, D] = sum_k weights[t, k] * y[dst[t*K + k]] +
+    sigmoid(shared_gate[t]) * shared[t] (shared None: no such term), fp32
+    sums; weights fp32 [T, K], shared_gate fp32 [T] (strided ok)."""
+    if y.is_cuda:
+        _require_streams()
+        out = torch.empty((weights.shape[0], y.shape[1]), dtype=y.dtype,
+                          device=y.device)
+        _streams.moe_combine(out, y, dst, weights, shared, shared_gate)
+        return out
+    T, K = weights.shape
+    out = (y[dst].view(T, K, -1).float() * weights[:, :, None]).sum(1)
+    if shared is not None:
+        out = out + torch.sigmoid(shared_gate)[:, None] * shared.float()
+    return out.to(y.dtype)

@@ -24,7 +24,7 @@ void relu2(torch::Tensor out, torch::Tensor in);
 void moe_topk_route(torch::Tensor weights, torch::Tensor idx,
                     torch::Tensor logits, c10::optional<torch::Tensor> dst,
                     c10::optional<torch::Tensor> counts, int64_t capacity,
-                    double scale);
+                    double scale, bool over_all);
 void add_rmsnorm_pair(torch::Tensor out1, c10::optional<torch::Tensor> out2,
                       torch::Tensor residual,
                       c10::optional<torch::Tensor> delta_a,

@@ -9,8 +9,8 @@
 //   rope_pairs        in-place rotation of a slice of every head, pairs
 //                     interleaved or half a slice apart
 //   xielu / relu2     feed-forward activations
-//   moe_topk_route    top-k experts + softmax over the chosen logits (times
-//                     a constant)
+//   moe_topk_route    top-k experts + softmax over the chosen logits or over
+//                     all of them (times a constant)
 //
 // One 256-thread block (4 waves) per token row for the row-wise kernels;
 // all arithmetic fp32, loads/stores in the activation type.
@@ -325,12 +325,13 @@ __global__ void moe_topk_route_kernel(float* __restrict__ weights,
                                       int32_t* __restrict__ idx,
                                       int64_t* __restrict__ dst,
                                       int32_t* __restrict__ counts,
-                                      const float* __restrict__ logits, int T,
-                                      int E, int K, int capacity,
-                                      float scale) {
+                                      const float* __restrict__ logits,
+                                      int64_t logits_rs, int T, int E, int K,
+                                      int capacity, float scale,
+                                      int over_all) {
   const int t = blockIdx.x * blockDim.x + threadIdx.x;
   if (t >= T) return;
-  const float* row = logits + (int64_t)t * E;
+  const float* row = logits + (int64_t)t * logits_rs;
   float* w = weights + (int64_t)t * K;
   int32_t* id = idx + (int64_t)t * K;
   uint64_t taken = 0;
@@ -356,6 +357,11 @@ __global__ void moe_topk_route_kernel(float* __restrict__ weights,
     w[k] = e;
     z += e;
   }
+  if (over_all) {
+    // the denominator of the softmax over every expert
+    z = 0.0f;
+    for (int e = 0; e < E; ++e) z += expf(row[e] - m);
+  }
   for (int k = 0; k < K; ++k) w[k] = w[k] / z * scale;
   // optional padded dispatch: row = expert * capacity + arrival rank (the
   // order inside an expert's segment carries no meaning: the gather back
@@ -372,9 +378,9 @@ __global__ void moe_topk_route_kernel(float* __restrict__ weights,
 void moe_topk_route(torch::Tensor weights, torch::Tensor idx,
                     torch::Tensor logits, c10::optional<torch::Tensor> dst,
                     c10::optional<torch::Tensor> counts, int64_t capacity,
-                    double scale) {
+                    double scale, bool over_all) {
   TORCH_CHECK(logits.is_cuda() && logits.dtype() == torch::kFloat32 &&
-              logits.is_contiguous() && logits.dim() == 2);
+              logits.dim() == 2 && logits.stride(1) == 1);
   const int T = logits.size(0), E = logits.size(1), K = weights.size(1);
   TORCH_CHECK(E <= 64 && K >= 1 && K <= E, "moe_topk_route: 1 <= k <= E <= 64");
   TORCH_CHECK(weights.is_contiguous() && weights.dtype() == torch::kFloat32 &&
@@ -395,8 +401,9 @@ void moe_topk_route(torch::Tensor weights, torch::Tensor idx,
                      (int32_t*)idx.data_ptr(),
                      dst.has_value() ? (int64_t*)dst->data_ptr() : nullptr,
                      dst.has_value() ? (int32_t*)counts->data_ptr() : nullptr,
-                     (const float*)logits.data_ptr(), T, E, K, (int)capacity,
-                     (float)scale);
+                     (const float*)logits.data_ptr(),
+                     (int64_t)logits.stride(0), T, E, K, (int)capacity,
+                     (float)scale, over_all ? 1 : 0);
   HIP_CHECK_KERNEL();
 }
 

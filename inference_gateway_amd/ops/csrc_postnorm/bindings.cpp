@@ -63,7 +63,8 @@ void qk_norm_rope_append(torch::Tensor qout, torch::Tensor proj,
                          c10::optional<torch::Tensor> knorm_w,
                          c10::optional<torch::Tensor> inv_freq, double mag,
                          double eps, int64_t heads, int64_t kv_heads,
-                         int64_t dim, int64_t vdim);
+                         int64_t dim, int64_t vdim, bool half,
+                         bool tied);
 void add_normed_rmsnorm(torch::Tensor out, torch::Tensor residual,
                         c10::optional<torch::Tensor> delta,
                         c10::optional<torch::Tensor> w_post,

@@ -77,7 +77,8 @@ void qk_norm_rope_append(torch::Tensor qout, torch::Tensor proj,
                          c10::optional<torch::Tensor> knorm_w,
                          c10::optional<torch::Tensor> inv_freq, double mag,
                          double eps, int64_t heads, int64_t kv_heads,
-                         int64_t dim, int64_t vdim);
+                         int64_t dim, int64_t vdim, bool half,
+                         bool tied);
 void moe_group_route(torch::Tensor weights, torch::Tensor idx,
                      torch::Tensor logits, torch::Tensor correction,
                      c10::optional<torch::Tensor> dst,

@@ -1,14 +1,16 @@
 // Query/key post-processing of a fused projection (gfx950): per-head RMS
-// norm, partial interleaved-pair rotation with scaled cos/sin, and the
-// append of keys and values to the paged caches, in one launch.
+// norm, partial pair rotation with scaled cos/sin, and the append of keys
+// and values to the paged caches, in one launch.
 //
 //   proj [T, H*N | G*N | G*P | ...]   (row stride of its own)
 //   x = head of q or k;  x <- x / sqrt(mean(x^2) + eps) * w      (w given)
-//   pairs (2i, 2i+1), i < R:  angle = position * inv_freq[i]
-//     (x_2i, x_2i+1) <- (x_2i c - x_2i+1 s, x_2i+1 c + x_2i s),
+//   pairs (a, b) = (2i, 2i+1), or HALF (i, i+R), i < R:
+//     angle = position * inv_freq[i]
+//     (x_a, x_b) <- (x_a c - x_b s, x_b c + x_a s),
 //     c = cos(angle) * mag, s = sin(angle) * mag
 //   q -> out [T, H*N];  k -> kcache [blocks, G, block, N] at slot;
-//   v -> vcache [blocks, G, block, P] at slot (copied)
+//   v -> vcache [blocks, G, block, P] at slot (copied); TIED: v is the key
+//   as projected, before norm and rotation, and proj has no value block
 //
 // One 256-thread workgroup per row; its four waves take the row's units in
 // turn: the H query heads, then the G key heads, then the G value heads.
@@ -47,14 +49,15 @@ struct Act2<uint16_t> {
 
 // PAIRED: every head starts on an even element and N, P are even, so a
 // pair is one aligned access
-template <typename T, bool PAIRED>
+template <typename T, bool PAIRED, bool HALF>
 __global__ __launch_bounds__(256) void qk_norm_rope_append_kernel(
     T* __restrict__ qout, const T* __restrict__ proj, int64_t proj_rs,
     const int32_t* __restrict__ positions,
     const int32_t* __restrict__ slot_mapping, T* __restrict__ kcache,
     T* __restrict__ vcache, const float* __restrict__ qnorm_w,
     const float* __restrict__ knorm_w, const float* __restrict__ inv_freq,
-    int R, float mag, float eps, int H, int G, int N, int P, int BS) {
+    int R, float mag, float eps, int H, int G, int N, int P, int BS,
+    int tied) {
   // cos | sin of the row's R angles, shared by all its heads
   extern __shared__ float cs_lds[];
   const int t = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
@@ -68,7 +71,7 @@ __global__ __launch_bounds__(256) void qk_norm_rope_append_kernel(
     cs_lds[R + i] = sinf(ang) * mag;
   }
   __syncthreads();
-  for (int unit = wave; unit < H + 2 * G; unit += 4) {
+  for (int unit = wave; unit < H + (tied ? G : 2 * G); unit += 4) {
     if (unit >= H + G) {
       // value head: plain copy into its page
       const int gv = unit - H - G;
@@ -89,6 +92,9 @@ __global__ __launch_bounds__(256) void qk_norm_rope_append_kernel(
     const T* src = row + (int64_t)unit * N;     // q heads then k heads
     T* dst = is_q ? qout + ((int64_t)t * H + unit) * N
                   : kcache + ((blk * G + (unit - H)) * BS + off) * N;
+    T* raw = !is_q && tied
+                 ? vcache + ((blk * G + (unit - H)) * BS + off) * P
+                 : nullptr;
     const float* w = is_q ? qnorm_w : knorm_w;
     const int npairs = (N + 1) / 2;
     // a head of up to 128 entries sits in one pair per lane; wider heads
@@ -123,13 +129,44 @@ __global__ __launch_bounds__(256) void qk_norm_rope_append_kernel(
         a = Act<T>::ld(src + d0);
         b = d1 < N ? Act<T>::ld(src + d1) : 0.0f;
       }
+      if (raw != nullptr) {
+        if (PAIRED) {
+          Act2<T>::st(raw + d0, a, b);
+        } else {
+          raw[d0] = src[d0];
+          if (d1 < N) raw[d1] = src[d1];
+        }
+      }
       a *= scale;
       b *= scale;
       if (w) {
         a *= w[d0];
         if (d1 < N) b *= w[d1];
       }
-      if (i < R) {
+      if (HALF) {
+        // this lane's two entries turn with entries R away (read again)
+        float* own[2] = {&a, &b};
+        float mate[2] = {0.0f, 0.0f};
+        if (PAIRED && !(R & 1)) {
+          if (d0 < 2 * R)
+            Act2<T>::ld(src + (d0 < R ? d0 + R : d0 - R), mate[0], mate[1]);
+        } else {
+#pragma unroll
+          for (int e = 0; e < 2; ++e) {
+            const int d = d0 + e;
+            if (d < 2 * R) mate[e] = Act<T>::ld(src + (d < R ? d + R : d - R));
+          }
+        }
+#pragma unroll
+        for (int e = 0; e < 2; ++e) {
+          const int d = d0 + e;
+          if (d >= 2 * R) continue;
+          const int m = d < R ? d + R : d - R, p = d < R ? d : d - R;
+          const float y = mate[e] * scale * (w ? w[m] : 1.0f);
+          const float c = cs_lds[p], s = cs_lds[R + p];
+          *own[e] = d < R ? *own[e] * c - y * s : *own[e] * c + y * s;
+        }
+      } else if (i < R) {
         const float c = cs_lds[i], s = cs_lds[R + i];
         const float ra = a * c - b * s, rb = b * c + a * s;
         a = ra;
@@ -152,10 +189,12 @@ void qk_norm_rope_append(torch::Tensor qout, torch::Tensor proj,
                          c10::optional<torch::Tensor> knorm_w,
                          c10::optional<torch::Tensor> inv_freq, double mag,
                          double eps, int64_t heads, int64_t kv_heads,
-                         int64_t dim, int64_t vdim) {
+                         int64_t dim, int64_t vdim, bool half, bool tied) {
   TORCH_CHECK(proj.is_cuda() && proj.dim() == 2 && proj.stride(1) == 1);
   const int T = proj.size(0), H = heads, G = kv_heads, N = dim, P = vdim;
-  TORCH_CHECK(proj.size(1) >= (int64_t)(H + G) * N + (int64_t)G * P);
+  TORCH_CHECK(proj.size(1) >=
+              (int64_t)(H + G) * N + (tied ? 0 : (int64_t)G * P));
+  TORCH_CHECK(!tied || P == N, "tied values have the keys' width");
   TORCH_CHECK(kcache.is_contiguous() && kcache.dim() == 4 &&
               vcache.is_contiguous() && vcache.dim() == 4 &&
               kcache.dtype() == proj.dtype() && vcache.dtype() == proj.dtype());
@@ -189,9 +228,9 @@ void qk_norm_rope_append(torch::Tensor qout, torch::Tensor proj,
   const bool paired =
       N % 2 == 0 && P % 2 == 0 && proj.stride(0) % 2 == 0 &&
       reinterpret_cast<uintptr_t>(proj.data_ptr()) % (2 * es) == 0;
-#define LAUNCH_QKR(PA)                                                        \
+#define LAUNCH_QKR(PA, HA)                                                        \
   hipLaunchKernelGGL(                                                         \
-      (qk_norm_rope_append_kernel<act_t, PA>), dim3(T), dim3(256),            \
+      (qk_norm_rope_append_kernel<act_t, PA, HA>), dim3(T), dim3(256),        \
       (size_t)(2 * R) * sizeof(float), stream,                                \
       (act_t*)qout.data_ptr(), (const act_t*)proj.data_ptr(),                 \
       (int64_t)proj.stride(0), (const int32_t*)positions.data_ptr(),          \
@@ -200,10 +239,12 @@ void qk_norm_rope_append(torch::Tensor qout, torch::Tensor proj,
       qnorm_w.has_value() ? (const float*)qnorm_w->data_ptr() : nullptr,      \
       knorm_w.has_value() ? (const float*)knorm_w->data_ptr() : nullptr,      \
       R ? (const float*)inv_freq->data_ptr() : nullptr, R, (float)mag,        \
-      (float)eps, H, G, N, P, BS)
+      (float)eps, H, G, N, P, BS, tied ? 1 : 0)
   IGW_DISPATCH_ACT(proj, {
-    if (paired) LAUNCH_QKR(true);
-    else LAUNCH_QKR(false);
+    if (paired && half) LAUNCH_QKR(true, true);
+    else if (paired) LAUNCH_QKR(true, false);
+    else if (half) LAUNCH_QKR(false, true);
+    else LAUNCH_QKR(false, false);
   });
 #undef LAUNCH_QKR
   HIP_CHECK_KERNEL();

@@ -1,0 +1,654 @@
+// Linear attention with one fixed decay per head (gfx950):
+//
+//   S_t = a_h S_{t-1} + k_t v_t^T,   o_t = S_t^T q_t        S [N, P] fp32
+//
+// q, k and v arrive as projected and pass silu here (SILU).  Two kernels:
+//
+//   step    any type and sizes, any number of rows: a workgroup keeps 64
+//           columns of S in registers (16 threads x 4 columns, 16 groups of
+//           key entries), so one decoded row is one load, one update and
+//           one store of the state with every access 16 bytes wide and all
+//           of them in flight together.
+//   chunks  bf16, N <= 128, MFMA: rows in chunks of C = 64.  With L rows
+//           in the chunk and S the memory before it,
+//             O[i] = a^{i+1} q_i S + sum_{j <= i} a^{i-j} (q_i.k_j) v_j
+//             S   <- a^L S + sum_j k_j (a^{L-1-j} v_j)^T
+//           A wave owns 16 value columns and keeps S for them as MFMA
+//           accumulators (fp32, in registers) across all chunks; S^T as the
+//           next product's operand, the weighted scores a^{i-j} (q.k) and
+//           the decayed values enter the matrix cores as a bf16 pair (high
+//           part + remainder), 16 mantissa bits, so recurrent state and
+//           attention weights are not rounded to bf16.
+//
+// The order of a contraction index is free as long as both operands agree
+// on it: accumulator tiles (lane = column, 4 consecutive rows) of two
+// neighbouring tiles are used directly as an operand of 32 contraction
+// entries, with lane group g holding entries {4g..4g+3, 16+4g..16+4g+3};
+// the other operand is fetched from LDS in that order (two 8-byte reads).
+//
+// Long prompts of few sequences are cut into segments: a first launch
+// leaves every segment's own contribution k (a^.. v)^T, a second one turns
+// these into the memory at each segment's start (and the sequence's final
+// state), and the main launch then runs all segments side by side.
+#include "../csrc_hybrid/act_types.h"
+
+namespace igw {
+
+typedef __attribute__((ext_vector_type(8))) short fd_short8;
+typedef __attribute__((ext_vector_type(4))) short fd_short4;
+typedef __attribute__((ext_vector_type(4))) float fd_float4;
+
+template <typename T>
+DEVINLINE float silu_for(float z) {
+  return z * sigmoid_for<T>(z);
+}
+
+// ---------------------------------------------------------------------------
+// step kernel
+// ---------------------------------------------------------------------------
+constexpr int FD_ROWS = 16;   // rows of q, k, v staged at a time
+constexpr int FD_PT = 64;     // value columns per workgroup
+
+template <typename T, int NPER, bool V4>
+__global__ __launch_bounds__(256) void fixed_decay_step_kernel(
+    float* __restrict__ out, const T* __restrict__ q, int64_t q_s0,
+    int64_t q_s1, const T* __restrict__ k, int64_t k_s0, int64_t k_s1,
+    const T* __restrict__ v, int64_t v_s0, int64_t v_s1,
+    const float* __restrict__ decay, float* __restrict__ state,
+    const int32_t* __restrict__ seqs, const int32_t* __restrict__ seq_cu,
+    const int32_t* __restrict__ seq_start,
+    const int32_t* __restrict__ seq_slots, int H, int G, int N, int P,
+    int silu) {
+  // q rows | k rows | v rows (FD_PT columns) | partial read-outs
+  extern __shared__ __attribute__((aligned(16))) float lds[];
+  float* lq = lds;
+  float* lk = lq + FD_ROWS * N;
+  float* lv = lk + FD_ROWS * N;
+  float* red = lv + FD_ROWS * FD_PT;      // [2][4 waves][FD_PT]
+  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
+  const int h = blockIdx.y, s = seqs[blockIdx.z];
+  const int g = h / (H / G);
+  const int r0 = seq_cu[s], r1 = seq_cu[s + 1];
+  if (r1 == r0) return;
+  const int c4 = (tid & 15) * 4, ng = tid >> 4;
+  const int p0 = blockIdx.x * FD_PT, p = p0 + c4;
+  const float a = decay[h];
+  const bool fresh = seq_start[s] == 0;
+  float* st = state + ((int64_t)seq_slots[s] * H + h) * N * P;
+
+  float S[NPER][4];
+#pragma unroll
+  for (int i = 0; i < NPER; ++i) {
+    const int n = i * 16 + ng;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) S[i][e] = 0.0f;
+    if (fresh || n >= N) continue;
+    if (V4) {
+      if (p < P) {
+        const float4 x = *(const float4*)(st + (int64_t)n * P + p);
+        S[i][0] = x.x;
+        S[i][1] = x.y;
+        S[i][2] = x.z;
+        S[i][3] = x.w;
+      }
+    } else {
+#pragma unroll
+      for (int e = 0; e < 4; ++e)
+        if (p + e < P) S[i][e] = st[(int64_t)n * P + p + e];
+    }
+  }
+  int par = 0;
+  for (int c0 = r0; c0 < r1; c0 += FD_ROWS) {
+    const int tc = min(FD_ROWS, r1 - c0);
+    if (c0 != r0) __syncthreads();    // everybody is done with the last rows
+    for (int i = tid; i < tc * N; i += 256) {
+      const int t = i / N, n = i - t * N;
+      const float x = Act<T>::ld(q + (c0 + t) * q_s0 + g * q_s1 + n);
+      const float y = Act<T>::ld(k + (c0 + t) * k_s0 + g * k_s1 + n);
+      lq[i] = silu ? silu_for<T>(x) : x;
+      lk[i] = silu ? silu_for<T>(y) : y;
+    }
+    for (int i = tid; i < tc * FD_PT; i += 256) {
+      const int t = i / FD_PT, c = i - t * FD_PT;
+      float x = 0.0f;
+      if (p0 + c < P) {
+        x = Act<T>::ld(v + (c0 + t) * v_s0 + h * v_s1 + p0 + c);
+        if (silu) x = silu_for<T>(x);
+      }
+      lv[i] = x;
+    }
+    __syncthreads();
+    for (int t = 0; t < tc; ++t) {
+      const float4 vv = *(const float4*)(lv + t * FD_PT + c4);
+      float o[4] = {0.0f, 0.0f, 0.0f, 0.0f};
+#pragma unroll
+      for (int i = 0; i < NPER; ++i) {
+        const int n = i * 16 + ng;
+        if (n >= N) continue;
+        const float kn = lk[t * N + n], qn = lq[t * N + n];
+        S[i][0] = a * S[i][0] + kn * vv.x;
+        S[i][1] = a * S[i][1] + kn * vv.y;
+        S[i][2] = a * S[i][2] + kn * vv.z;
+        S[i][3] = a * S[i][3] + kn * vv.w;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) o[e] += qn * S[i][e];
+      }
+      // sum over the four groups of a wave, then over the waves.  Two
+      // buffers in turn: a buffer is written again only after the next
+      // row's barrier, which its readers reach when they have read it
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        o[e] += __shfl_xor(o[e], 16, 64);
+        o[e] += __shfl_xor(o[e], 32, 64);
+      }
+      float* rb = red + par * 4 * FD_PT;
+      if (lane < 16)
+        *(float4*)(rb + wave * FD_PT + c4) =
+            make_float4(o[0], o[1], o[2], o[3]);
+      __syncthreads();
+      if (tid < FD_PT && p0 + tid < P)
+        out[((int64_t)(c0 + t) * H + h) * P + p0 + tid] =
+            rb[tid] + rb[FD_PT + tid] + rb[2 * FD_PT + tid] +
+            rb[3 * FD_PT + tid];
+      par ^= 1;
+    }
+  }
+#pragma unroll
+  for (int i = 0; i < NPER; ++i) {
+    const int n = i * 16 + ng;
+    if (n >= N) continue;
+    if (V4) {
+      if (p < P)
+        *(float4*)(st + (int64_t)n * P + p) =
+            make_float4(S[i][0], S[i][1], S[i][2], S[i][3]);
+    } else {
+#pragma unroll
+      for (int e = 0; e < 4; ++e)
+        if (p + e < P) st[(int64_t)n * P + p + e] = S[i][e];
+    }
+  }
+}
+
+// ---------------------------------------------------------------------------
+// chunk kernel
+// ---------------------------------------------------------------------------
+constexpr int FD_C = 64;      // rows per chunk
+
+// 8 floats -> bf16 high parts and bf16 remainders
+DEVINLINE void split_pair(const float* x, fd_short8& hi, fd_short8& lo) {
+#pragma unroll
+  for (int e = 0; e < 8; ++e) {
+    const uint16_t b = f32_to_bf16(x[e]);
+    hi[e] = (short)b;
+    lo[e] = (short)f32_to_bf16(x[e] - bf16_to_f32(b));
+  }
+}
+
+DEVINLINE fd_float4 mfma_bf16(fd_short8 a, fd_short8 b, fd_float4 c) {
+  return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0);
+}
+
+// two 8-byte LDS reads: entries {4g..4g+3} and {16+4g..16+4g+3} of a row
+DEVINLINE fd_short8 frag_perm(const uint16_t* row, int g) {
+  const fd_short4 a = *(const fd_short4*)(row + 4 * g);
+  const fd_short4 b = *(const fd_short4*)(row + 16 + 4 * g);
+  return fd_short8{a[0], a[1], a[2], a[3], b[0], b[1], b[2], b[3]};
+}
+
+// segment table, int32 [5][nseg]: first row, end row, sequence, first
+// segment of its sequence (0/1), last segment of its sequence (0/1)
+template <int NP, int NW, bool VEC, bool STATE_ONLY>
+__global__ __launch_bounds__(NW * 64) void fixed_decay_chunk_kernel(
+    float* __restrict__ out, const uint16_t* __restrict__ q, int64_t q_s0,
+    int64_t q_s1, const uint16_t* __restrict__ k, int64_t k_s0, int64_t k_s1,
+    const uint16_t* __restrict__ v, int64_t v_s0, int64_t v_s1,
+    const float* __restrict__ decay, float* __restrict__ state,
+    float* __restrict__ work, const int32_t* __restrict__ segs, int nseg,
+    const int32_t* __restrict__ seq_start,
+    const int32_t* __restrict__ seq_slots, int H, int G, int N, int P,
+    int silu) {
+  constexpr int NTILE = NP / 16;
+  constexpr int RS = NP + 8;         // LDS row stride of q and k
+  constexpr int CS = FD_C + 8;       // ... of the transposed k and v
+  constexpr int PT = NW * 16;
+  constexpr int NQ = NP / 8 / NW > 0 ? NP / 8 / NW : 1;   // pieces per thread
+  __shared__ __attribute__((aligned(16))) uint16_t qs[STATE_ONLY ? 8
+                                                                 : FD_C * RS];
+  __shared__ __attribute__((aligned(16))) uint16_t ks[STATE_ONLY ? 8
+                                                                 : FD_C * RS];
+  __shared__ __attribute__((aligned(16))) uint16_t kt[NP * CS];
+  __shared__ __attribute__((aligned(16))) uint16_t vt[PT * CS];
+  // weighted scores as operand fragments: [row tile][k step][hi|lo][lane]
+  __shared__ __attribute__((aligned(16)))
+  uint16_t af[STATE_ONLY ? 8 : 4 * 2 * 2 * 64 * 8];
+  __shared__ float pw[FD_C + 1];
+  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
+  const int l16 = lane & 15, g4 = lane >> 4;
+  const int sg = blockIdx.z, h = blockIdx.y;
+  const int row0 = segs[sg], row1 = segs[nseg + sg];
+  const int seq = segs[2 * nseg + sg];
+  const bool first = segs[3 * nseg + sg] != 0;
+  const bool last = segs[4 * nseg + sg] != 0;
+  const int kh = h / (H / G);
+  const float a = decay[h];
+  if (tid <= FD_C) pw[tid] = tid == 0 ? 1.0f : powf(a, (float)tid);
+  const int p0 = blockIdx.x * PT;
+  const int pc = p0 + wave * 16 + l16;     // this lane's value column
+  float* st = state + ((int64_t)seq_slots[seq] * H + h) * N * P;
+  float* wk = work == nullptr
+                  ? nullptr
+                  : work + ((int64_t)sg * H + h) * N * P;
+
+  // S tiles: column pc, rows 16 nt + 4 g4 + r
+  fd_float4 S[NTILE];
+  {
+    const float* src = nullptr;
+    if (!STATE_ONLY) {
+      if (wk != nullptr) src = wk;                 // memory at its start
+      else if (!(first && seq_start[seq] == 0)) src = st;
+    }
+#pragma unroll
+    for (int nt = 0; nt < NTILE; ++nt)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int n = nt * 16 + g4 * 4 + r;
+        S[nt][r] = (src != nullptr && n < N && pc < P)
+                       ? src[(int64_t)n * P + pc]
+                       : 0.0f;
+      }
+  }
+
+  // staging: lane = row of the chunk, a thread takes NQ pieces of 8 key
+  // entries (piece = wave + NW * i) and two pieces of 8 value columns
+  ushort8 qr[NQ], kr[NQ], vr[2];
+  auto piece = [&](const uint16_t* base, int width, int c8, bool ok) {
+    ushort8 x;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) x.v[e] = 0;
+    if (!ok) return x;
+    if (VEC) {
+      if (c8 < width) x = *(const ushort8*)(base + c8);
+    } else {
+#pragma unroll
+      for (int e = 0; e < 8; ++e)
+        if (c8 + e < width) x.v[e] = base[c8 + e];
+    }
+    return x;
+  };
+  auto fetch = [&](int c0) {
+    const int64_t row = c0 + lane;
+    const bool ok = row < row1;
+#pragma unroll
+    for (int i = 0; i < NQ; ++i) {
+      const int c8 = (wave + NW * i) * 8;
+      const bool in = ok && c8 < NP;
+      kr[i] = piece(k + row * k_s0 + kh * k_s1, N, c8, in);
+      if (!STATE_ONLY) qr[i] = piece(q + row * q_s0 + kh * q_s1, N, c8, in);
+    }
+#pragma unroll
+    for (int i = 0; i < 2; ++i) {
+      const int c8 = (wave + NW * i) * 8;
+      vr[i] = piece(v + row * v_s0 + h * v_s1 + p0, P - p0, c8, ok);
+    }
+  };
+  auto act8 = [&](ushort8 x) {
+    if (silu) {
+#pragma unroll
+      for (int e = 0; e < 8; ++e)
+        x.v[e] = f32_to_bf16(silu_for<uint16_t>(bf16_to_f32(x.v[e])));
+    }
+    return x;      // silu(0) = 0: padding stays zero
+  };
+
+  fetch(row0);
+  for (int c0 = row0; c0 < row1; c0 += FD_C) {
+    const int L = min(FD_C, row1 - c0);
+#pragma unroll
+    for (int i = 0; i < NQ; ++i) {
+      const int c8 = (wave + NW * i) * 8;
+      if (c8 < NP) {
+        const ushort8 kk = act8(kr[i]);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) kt[(c8 + e) * CS + lane] = kk.v[e];
+        if (!STATE_ONLY) {
+          *(ushort8*)(ks + lane * RS + c8) = kk;
+          *(ushort8*)(qs + lane * RS + c8) = act8(qr[i]);
+        }
+      }
+    }
+#pragma unroll
+    for (int i = 0; i < 2; ++i) {
+      const int c8 = (wave + NW * i) * 8;
+      const ushort8 vv = act8(vr[i]);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) vt[(c8 + e) * CS + lane] = vv.v[e];
+    }
+    __syncthreads();
+    if (c0 + FD_C < row1) fetch(c0 + FD_C);
+
+    if (!STATE_ONLY) {
+      // weighted scores of (16 rows i) x (32 rows j), transposed product
+      // K Q^T: lane column = i, accumulator rows = j
+      for (int un = wave; un < 8; un += NW) {
+        const int it = un & 3, kst = un >> 2;
+        if (kst * 32 > it * 16 + 15) continue;     // all j > i
+        fd_float4 c[2];
+#pragma unroll
+        for (int x = 0; x < 2; ++x) c[x] = fd_float4{0, 0, 0, 0};
+#pragma unroll
+        for (int ns = 0; ns < NP / 32; ++ns) {
+          const fd_short8 b = *(const fd_short8*)(
+              qs + (it * 16 + l16) * RS + ns * 32 + g4 * 8);
+#pragma unroll
+          for (int x = 0; x < 2; ++x) {
+            const fd_short8 aa = *(const fd_short8*)(
+                ks + (kst * 32 + x * 16 + l16) * RS + ns * 32 + g4 * 8);
+            c[x] = mfma_bf16(aa, b, c[x]);
+          }
+        }
+        float w[8];
+        const int i = it * 16 + l16;
+#pragma unroll
+        for (int x = 0; x < 2; ++x)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) {
+            const int j = kst * 32 + x * 16 + g4 * 4 + r;
+            w[x * 4 + r] = j <= i ? pw[i - j] * c[x][r] : 0.0f;
+          }
+        fd_short8 hi, lo;
+        split_pair(w, hi, lo);
+        uint16_t* f = af + ((it * 2 + kst) * 2 * 64 + lane) * 8;
+        *(fd_short8*)f = hi;
+        *(fd_short8*)(f + 64 * 8) = lo;
+      }
+      // read-out of the memory before the chunk: O = a^{i+1} Q S
+      fd_float4 acc[4];
+#pragma unroll
+      for (int it = 0; it < 4; ++it) acc[it] = fd_float4{0, 0, 0, 0};
+#pragma unroll
+      for (int ns = 0; ns < NP / 32; ++ns) {
+        float x[8];
+#pragma unroll
+        for (int e = 0; e < 8; ++e) x[e] = S[2 * ns + (e >> 2)][e & 3];
+        fd_short8 hi, lo;
+        split_pair(x, hi, lo);
+#pragma unroll
+        for (int it = 0; it < 4; ++it) {
+          const fd_short8 aa =
+              frag_perm(qs + (it * 16 + l16) * RS + ns * 32, g4);
+          acc[it] = mfma_bf16(aa, hi, acc[it]);
+          acc[it] = mfma_bf16(aa, lo, acc[it]);
+        }
+      }
+#pragma unroll
+      for (int it = 0; it < 4; ++it)
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+          acc[it][r] *= pw[it * 16 + g4 * 4 + r + 1];
+      __syncthreads();     // score fragments
+      fd_short8 vb[2];
+#pragma unroll
+      for (int kst = 0; kst < 2; ++kst)
+        vb[kst] = frag_perm(vt + (wave * 16 + l16) * CS + kst * 32, g4);
+#pragma unroll
+      for (int it = 0; it < 4; ++it)
+#pragma unroll
+        for (int kst = 0; kst < 2; ++kst) {
+          if (kst * 32 > it * 16 + 15) continue;
+          const uint16_t* f = af + ((it * 2 + kst) * 2 * 64 + lane) * 8;
+          acc[it] = mfma_bf16(*(const fd_short8*)f, vb[kst], acc[it]);
+          acc[it] = mfma_bf16(*(const fd_short8*)(f + 64 * 8), vb[kst],
+                              acc[it]);
+        }
+      if (pc < P) {
+#pragma unroll
+        for (int it = 0; it < 4; ++it)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) {
+            const int i = it * 16 + g4 * 4 + r;
+            if (i < L) out[((int64_t)(c0 + i) * H + h) * P + pc] = acc[it][r];
+          }
+      }
+    }
+    // memory after the chunk
+    const float aL = pw[L];
+#pragma unroll
+    for (int nt = 0; nt < NTILE; ++nt) S[nt] *= aL;
+#pragma unroll
+    for (int js = 0; js < 2; ++js) {
+      const fd_short8 raw = *(const fd_short8*)(
+          vt + (wave * 16 + l16) * CS + js * 32 + g4 * 8);
+      float x[8];
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        const int j = js * 32 + g4 * 8 + e;
+        x[e] = j < L ? bf16_to_f32((uint16_t)raw[e]) * pw[L - 1 - j] : 0.0f;
+      }
+      fd_short8 hi, lo;
+      split_pair(x, hi, lo);
+#pragma unroll
+      for (int nt = 0; nt < NTILE; ++nt) {
+        const fd_short8 aa = *(const fd_short8*)(
+            kt + (nt * 16 + l16) * CS + js * 32 + g4 * 8);
+        S[nt] = mfma_bf16(aa, hi, S[nt]);
+        S[nt] = mfma_bf16(aa, lo, S[nt]);
+      }
+    }
+    __syncthreads();       // the staged rows are free again
+  }
+  float* dst = STATE_ONLY ? wk : (last && wk == nullptr ? st : nullptr);
+  if (dst != nullptr && pc < P) {
+#pragma unroll
+    for (int nt = 0; nt < NTILE; ++nt)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int n = nt * 16 + g4 * 4 + r;
+        if (n < N) dst[(int64_t)n * P + pc] = S[nt][r];
+      }
+  }
+}
+
+// work[segment] holds the segment's own contribution; becomes the memory at
+// the segment's start, in order, and the slot gets the final one.
+// seg_first[i] .. seg_first[i + 1] are the segments of the i-th sequence.
+__global__ __launch_bounds__(256) void fixed_decay_carry_kernel(
+    float* __restrict__ work, float* __restrict__ state,
+    const float* __restrict__ decay, const int32_t* __restrict__ segs,
+    int nseg, const int32_t* __restrict__ seg_first,
+    const int32_t* __restrict__ seq_start,
+    const int32_t* __restrict__ seq_slots, int H, int64_t NP_) {
+  const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
+  if (i >= NP_) return;
+  const int h = blockIdx.y;
+  const int s0 = seg_first[blockIdx.z], s1 = seg_first[blockIdx.z + 1];
+  if (s0 == s1) return;
+  const int seq = segs[2 * nseg + s0];
+  const float a = decay[h];
+  float* st = state + ((int64_t)seq_slots[seq] * H + h) * NP_ + i;
+  float x = seq_start[seq] == 0 ? 0.0f : *st;
+  for (int s = s0; s < s1; ++s) {
+    float* w = work + ((int64_t)s * H + h) * NP_ + i;
+    const float own = *w;
+    *w = x;
+    x = powf(a, (float)(segs[nseg + s] - segs[s])) * x + own;
+  }
+  *st = x;
+}
+
+// ---------------------------------------------------------------------------
+int64_t fixed_decay_chunk_keys() { return 128; }   // widest N of the chunks
+
+static void fd_check(const torch::Tensor& out, const torch::Tensor& q,
+                     const torch::Tensor& k, const torch::Tensor& v,
+                     const torch::Tensor& decay, const torch::Tensor& state) {
+  TORCH_CHECK(v.is_cuda() && v.dim() == 3 && v.stride(2) == 1 &&
+              q.dim() == 3 && q.stride(2) == 1 && k.dim() == 3 &&
+              k.stride(2) == 1 && q.dtype() == v.dtype() &&
+              k.dtype() == v.dtype() && q.sizes() == k.sizes() &&
+              q.size(0) == v.size(0));
+  const int64_t T = v.size(0), H = v.size(1), P = v.size(2);
+  const int64_t G = q.size(1), N = q.size(2);
+  TORCH_CHECK(G >= 1 && H % G == 0 && N >= 1 && P >= 1);
+  TORCH_CHECK(out.dtype() == torch::kFloat32 && out.is_contiguous() &&
+              out.numel() == T * H * P);
+  TORCH_CHECK(decay.dtype() == torch::kFloat32 && decay.is_contiguous() &&
+              decay.numel() == H);
+  TORCH_CHECK(state.dtype() == torch::kFloat32 && state.is_contiguous() &&
+              state.dim() == 2 && state.size(1) == H * N * P,
+              "memory slot width must be heads * keys * values");
+}
+
+static void fd_check_seqs(const torch::Tensor& seq_start,
+                          const torch::Tensor& seq_slots) {
+  TORCH_CHECK(seq_start.dtype() == torch::kInt32 &&
+              seq_slots.dtype() == torch::kInt32 &&
+              seq_start.is_contiguous() && seq_slots.is_contiguous() &&
+              seq_start.numel() == seq_slots.numel());
+}
+
+void fixed_decay_step(torch::Tensor out, torch::Tensor q, torch::Tensor k,
+                      torch::Tensor v, torch::Tensor decay,
+                      torch::Tensor state, torch::Tensor seqs,
+                      torch::Tensor seq_cu, torch::Tensor seq_start,
+                      torch::Tensor seq_slots, bool silu) {
+  fd_check(out, q, k, v, decay, state);
+  fd_check_seqs(seq_start, seq_slots);
+  const int H = v.size(1), P = v.size(2), G = q.size(1), N = q.size(2);
+  const int S = seqs.numel();
+  TORCH_CHECK(seqs.dtype() == torch::kInt32 && seqs.is_contiguous() &&
+              seq_cu.dtype() == torch::kInt32 &&
+              seq_cu.numel() == seq_start.numel() + 1);
+  TORCH_CHECK(N <= 512, "key width above 512 is not supported");
+  if (v.size(0) == 0 || S == 0) return;
+  hipStream_t stream = at::cuda::getCurrentCUDAStream();
+  const dim3 grid((P + FD_PT - 1) / FD_PT, H, S);
+  const size_t shmem =
+      sizeof(float) * (2 * (size_t)FD_ROWS * N + FD_ROWS * FD_PT +
+                       2 * 4 * FD_PT);
+  const bool v4 = P % 4 == 0 &&
+                  reinterpret_cast<uintptr_t>(state.data_ptr()) % 16 == 0;
+#define FD_STEP(NPERV, V4V)                                                   \
+  do {                                                                        \
+    auto kern = fixed_decay_step_kernel<act_t, NPERV, V4V>;                   \
+    if (shmem > 64 * 1024)                                                    \
+      (void)hipFuncSetAttribute((const void*)kern,                            \
+                                hipFuncAttributeMaxDynamicSharedMemorySize,   \
+                                (int)shmem);                                  \
+    hipLaunchKernelGGL(                                                       \
+        kern, grid, dim3(256), shmem, stream, (float*)out.data_ptr(),         \
+        (const act_t*)q.data_ptr(), (int64_t)q.stride(0),                     \
+        (int64_t)q.stride(1), (const act_t*)k.data_ptr(),                     \
+        (int64_t)k.stride(0), (int64_t)k.stride(1),                           \
+        (const act_t*)v.data_ptr(), (int64_t)v.stride(0),                     \
+        (int64_t)v.stride(1), (const float*)decay.data_ptr(),                 \
+        (float*)state.data_ptr(), (const int32_t*)seqs.data_ptr(),            \
+        (const int32_t*)seq_cu.data_ptr(),                                    \
+        (const int32_t*)seq_start.data_ptr(),                                 \
+        (const int32_t*)seq_slots.data_ptr(), H, G, N, P, silu ? 1 : 0);      \
+  } while (0)
+#define FD_STEP_N(NPERV)                                                      \
+  do {                                                                        \
+    if (v4) FD_STEP(NPERV, true);                                             \
+    else FD_STEP(NPERV, false);                                               \
+  } while (0)
+  IGW_DISPATCH_ACT(v, {
+    if (N <= 16) FD_STEP_N(1);
+    else if (N <= 32) FD_STEP_N(2);
+    else if (N <= 64) FD_STEP_N(4);
+    else if (N <= 128) FD_STEP_N(8);
+    else if (N <= 256) FD_STEP_N(16);
+    else FD_STEP_N(32);
+  });
+#undef FD_STEP_N
+#undef FD_STEP
+  (void)hipGetLastError();   // a refused attribute must not poison the check
+  HIP_CHECK_KERNEL();
+}
+
+// segs int32 [5, nseg] (see the kernel); work fp32 [nseg, H, N, P] when the
+// prompts are cut into segments that run side by side, with seg_first int32
+// [sequences + 1]; without work every sequence is one segment.
+void fixed_decay_chunks(torch::Tensor out, torch::Tensor q, torch::Tensor k,
+                        torch::Tensor v, torch::Tensor decay,
+                        torch::Tensor state, torch::Tensor segs,
+                        c10::optional<torch::Tensor> work,
+                        c10::optional<torch::Tensor> seg_first,
+                        torch::Tensor seq_start, torch::Tensor seq_slots,
+                        bool silu) {
+  fd_check(out, q, k, v, decay, state);
+  fd_check_seqs(seq_start, seq_slots);
+  const int H = v.size(1), P = v.size(2), G = q.size(1), N = q.size(2);
+  TORCH_CHECK(v.scalar_type() == torch::kBFloat16 &&
+              N <= fixed_decay_chunk_keys());
+  TORCH_CHECK(segs.dtype() == torch::kInt32 && segs.is_contiguous() &&
+              segs.dim() == 2 && segs.size(0) == 5);
+  const int nseg = segs.size(1);
+  TORCH_CHECK(work.has_value() == seg_first.has_value());
+  if (work.has_value())
+    TORCH_CHECK(work->dtype() == torch::kFloat32 && work->is_contiguous() &&
+                work->numel() == (int64_t)nseg * H * N * P &&
+                seg_first->dtype() == torch::kInt32 &&
+                seg_first->is_contiguous());
+  if (v.size(0) == 0 || nseg == 0) return;
+  hipStream_t stream = at::cuda::getCurrentCUDAStream();
+  const int nw = P <= 64 ? 4 : 8;
+  const dim3 grid((P + nw * 16 - 1) / (nw * 16), H, nseg);
+  auto aligned = [](const torch::Tensor& t) {
+    return reinterpret_cast<uintptr_t>(t.data_ptr()) % 16 == 0 &&
+           t.stride(0) % 8 == 0 && t.stride(1) % 8 == 0;
+  };
+  const bool vec = N % 8 == 0 && P % 8 == 0 && aligned(q) && aligned(k) &&
+                   aligned(v);
+#define FD_CHUNK(NPV, NWV, VECV, SOV)                                         \
+  hipLaunchKernelGGL(                                                         \
+      (fixed_decay_chunk_kernel<NPV, NWV, VECV, SOV>), grid, dim3(NWV * 64),  \
+      0, stream, (float*)out.data_ptr(), (const uint16_t*)q.data_ptr(),       \
+      (int64_t)q.stride(0), (int64_t)q.stride(1),                             \
+      (const uint16_t*)k.data_ptr(), (int64_t)k.stride(0),                    \
+      (int64_t)k.stride(1), (const uint16_t*)v.data_ptr(),                    \
+      (int64_t)v.stride(0), (int64_t)v.stride(1),                             \
+      (const float*)decay.data_ptr(), (float*)state.data_ptr(),               \
+      work.has_value() ? (float*)work->data_ptr() : nullptr,                  \
+      (const int32_t*)segs.data_ptr(), nseg,                                  \
+      (const int32_t*)seq_start.data_ptr(),                                   \
+      (const int32_t*)seq_slots.data_ptr(), H, G, N, P, silu ? 1 : 0)
+#define FD_CHUNK_V(NPV, NWV, SOV)                                             \
+  do {                                                                        \
+    if (vec) FD_CHUNK(NPV, NWV, true, SOV);                                   \
+    else FD_CHUNK(NPV, NWV, false, SOV);                                      \
+  } while (0)
+#define FD_CHUNK_N(NPV, SOV)                                                  \
+  do {                                                                        \
+    if (nw == 4) FD_CHUNK_V(NPV, 4, SOV);                                     \
+    else FD_CHUNK_V(NPV, 8, SOV);                                             \
+  } while (0)
+#define FD_CHUNK_ALL(SOV)                                                     \
+  do {                                                                        \
+    if (N <= 32) FD_CHUNK_N(32, SOV);                                         \
+    else if (N <= 64) FD_CHUNK_N(64, SOV);                                    \
+    else FD_CHUNK_N(128, SOV);                                                \
+  } while (0)
+  if (work.has_value()) {
+    FD_CHUNK_ALL(true);
+    HIP_CHECK_KERNEL();
+    const int64_t np = (int64_t)N * P;
+    hipLaunchKernelGGL(
+        fixed_decay_carry_kernel,
+        dim3((unsigned)((np + 255) / 256), H, seg_first->numel() - 1),
+        dim3(256), 0, stream, (float*)work->data_ptr(),
+        (float*)state.data_ptr(), (const float*)decay.data_ptr(),
+        (const int32_t*)segs.data_ptr(), nseg,
+        (const int32_t*)seg_first->data_ptr(),
+        (const int32_t*)seq_start.data_ptr(),
+        (const int32_t*)seq_slots.data_ptr(), H, np);
+    HIP_CHECK_KERNEL();
+  }
+  FD_CHUNK_ALL(false);
+#undef FD_CHUNK_ALL
+#undef FD_CHUNK_N
+#undef FD_CHUNK_V
+#undef FD_CHUNK
+  HIP_CHECK_KERNEL();
+}
+
+}  // namespace igw

@@ -260,18 +260,20 @@ def softcap_attention_ref(q, kcache, vcache, block_table, row_seq,
 
 def qk_norm_rope_append_ref(proj, positions, slot_mapping, kcache, vcache,
                             qnorm_w, knorm_w, inv_freq, mag, eps, heads,
-                            kv_heads, dim, vdim):
+                            kv_heads, dim, vdim, half=False, tied=False):
     """proj [T, heads*dim | kv_heads*dim | kv_heads*vdim | ...]: every
     query and key head is RMS-normed over its dim entries (weights [dim]
-    shared by the heads; None = no norm), then pairs (2i, 2i+1) of its
-    first 2*len(inv_freq) entries turn by position * inv_freq[i] with cos
-    and sin times `mag` (inv_freq None = no rotation).  Keys and values
-    go to the paged caches; the queries are returned [T, heads*dim]."""
+    shared by the heads; None = no norm), then pairs (2i, 2i+1), or with
+    `half` (i, i + len(inv_freq)), of its first 2*len(inv_freq) entries
+    turn by position * inv_freq[i] with cos and sin times `mag` (inv_freq
+    None = no rotation).  Keys and values (`tied`: the projected keys) go
+    to the paged caches; the queries are returned [T, heads*dim]."""
     T = proj.shape[0]
     nq, nk = heads * dim, kv_heads * dim
     q = proj[:, :nq].float().reshape(T, heads, dim)
     k = proj[:, nq:nq + nk].float().reshape(T, kv_heads, dim)
-    v = proj[:, nq + nk:nq + nk + kv_heads * vdim]
+    v = proj[:, nq:nq + nk] if tied \
+        else proj[:, nq + nk:nq + nk + kv_heads * vdim]
 
     def prep(x, w):
         if w is not None:
@@ -281,8 +283,12 @@ def qk_norm_rope_append_ref(proj, positions, slot_mapping, kcache, vcache,
             ang = positions.float()[:, None] * inv_freq.float()[None, :]
             c = (torch.cos(ang) * mag)[:, None, :]
             s = (torch.sin(ang) * mag)[:, None, :]
-            a, b = x[..., 0:2 * R:2], x[..., 1:2 * R:2]
-            rot = torch.stack([a * c - b * s, b * c + a * s], -1)
+            if half:
+                a, b = x[..., :R], x[..., R:2 * R]
+            else:
+                a, b = x[..., 0:2 * R:2], x[..., 1:2 * R:2]
+            rot = [a * c - b * s, b * c + a * s]
+            rot = torch.cat(rot, -1) if half else torch.stack(rot, -1)
             x = torch.cat([rot.reshape(T, x.shape[1], 2 * R),
                            x[..., 2 * R:]], -1)
         return x
@@ -391,3 +397,62 @@ def rmsnorm_pair_mean_ref(a, b, wa, wb, eps):
     ya = af * torch.rsqrt((af * af).mean(-1, keepdim=True) + eps) * wa
     yb = bf * torch.rsqrt((bf * bf).mean(-1, keepdim=True) + eps) * wb
     return (0.5 * (ya + yb)).to(a.dtype)
+
+
+def stream_step_ref(streams, y, mix, outw, inw, norm_w, eps, out_dtype):
+    """Residual streams [T, B, D]: new stream t = sum_b mix[b, t] X_b +
+    outw[t] y (y None: unchanged); RMS norm of sum_t inw[t] X_t times
+    norm_w."""
+    if y is not None:
+        streams = (torch.matmul(mix.t(), streams)
+                   + outw[None, :, None] * y.float()[:, None, :])
+    u = (streams * inw[None, :, None]).sum(1)
+    h = u * torch.rsqrt((u * u).mean(-1, keepdim=True) + eps) * norm_w
+    return streams, h.to(out_dtype)
+
+
+def latent_rope_append_ref(x, positions, slot_mapping, cache, norm_w,
+                           inv_freq, eps, heads, dim, rot_dim, kv_rank,
+                           half, mag):
+    """x [T, heads*(dim+rot_dim) | kv_rank | rot_dim]: query heads' last
+    rot_dim entries rotated in place; normed latent and rotated shared key
+    appended to the paged rows."""
+    from .torch_ref import _rotate
+
+    T, nq = x.shape[0], heads * (dim + rot_dim)
+    n2 = 2 * inv_freq.numel()
+    q = x[:, :nq].view(T, heads, dim + rot_dim)
+    r = q[:, :, dim:dim + n2].float().reshape(T * heads, n2)
+    q[:, :, dim:dim + n2] = _rotate(
+        r, positions.repeat_interleave(heads), inv_freq, half,
+        mag).view(T, heads, n2).to(x.dtype)
+    c = x[:, nq:nq + kv_rank].float()
+    c = c * torch.rsqrt((c * c).mean(-1, keepdim=True) + eps) * norm_w
+    kr = x[:, nq + kv_rank:].float().clone()
+    kr[:, :n2] = _rotate(kr[:, :n2], positions, inv_freq, half, mag)
+    cache.view(-1, cache.shape[-1])[slot_mapping.long()] = torch.cat(
+        [c, kr], -1).to(cache.dtype)
+
+
+def fixed_decay_scan_ref(q, k, v, decay, state, seq_cu, seq_start,
+                         seq_slots, silu):
+    """S <- decay_h S + k_t v_t^T, o_t = S^T q_t per (sequence, head),
+    with silu on q, k, v first when asked."""
+    T, H, P = v.shape
+    G, N = q.shape[1], q.shape[2]
+    q, k, v = q.float(), k.float(), v.float()
+    if silu:
+        q, k, v = F.silu(q), F.silu(k), F.silu(v)
+    q, k = (x.repeat_interleave(H // G, 1) for x in (q, k))
+    a = decay.view(H, 1, 1)
+    out = torch.empty((T, H, P), dtype=torch.float32, device=v.device)
+    for r0, r1, st, sl in _seqs(seq_cu, seq_start, seq_slots):
+        if r1 == r0:
+            continue
+        S = (state[sl].view(H, N, P).clone() if st > 0 else torch.zeros(
+            (H, N, P), dtype=torch.float32, device=v.device))
+        for t in range(r0, r1):
+            S = a * S + k[t][:, :, None] * v[t][:, None, :]
+            out[t] = (S * q[t][:, :, None]).sum(1)
+        state[sl] = S.reshape(-1)
+    return out

@@ -462,9 +462,13 @@ def relu2_ref(z):
     return (r * r).to(z.dtype)
 
 
-def moe_topk_route_ref(logits, top_k):
-    """Top-k experts by logit and the softmax over just those k."""
+def moe_topk_route_ref(logits, top_k, over_all=False):
+    """Top-k experts by logit and the softmax over just those k, or
+    (over_all) their entries of the softmax over every expert."""
     w, idx = torch.topk(logits, top_k, dim=-1)
+    if over_all:
+        return (torch.softmax(logits, dim=-1).gather(1, idx),
+                idx.to(torch.int32))
     return torch.softmax(w, dim=-1), idx.to(torch.int32)
 
 

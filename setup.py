@@ -42,6 +42,15 @@ postnorm_sources = [str(PN / "bindings.cpp")] + [
     str(REC / f) for f in ("qk_rope_append.hip", "sandwich_ops.hip",
                            "softcap_attn.hip", "softcap_attn_mfma.hip")]
 
+# the multi-stream extension: its own kernels plus the attention, row and
+# router kernels its models launch
+STR = ROOT / "inference_gateway_amd" / "ops" / "csrc_streams"
+streams_sources = [str(STR / "bindings.cpp")] + _hip_sources(STR) + [
+    str(HYB / f) for f in ("hybrid_ops.hip", "latent_attn.hip",
+                           "latent_attn_mfma.hip", "parallel_ops.hip")] + [
+    str(REC / f) for f in ("qk_rope_append.hip", "recurrent_ops.hip",
+                           "softcap_attn.hip", "softcap_attn_mfma.hip")]
+
 # packed-fp32 instruction selection is switched off for all device code
 HIPCC_FLAGS = [
     "-O3",
@@ -60,7 +69,7 @@ def _ext(name, srcs):
     )
 
 
-# IGW_BUILD_EXT=hybrid|kernels|postnorm|recurrent builds just one extension (a
+# IGW_BUILD_EXT=hybrid|kernels|postnorm|recurrent|streams builds just one extension (a
 # process that serves one model family compiles only what it loads);
 # default: all
 _which = os.environ.get("IGW_BUILD_EXT", "all")
@@ -77,6 +86,9 @@ if _which in ("all", "recurrent"):
 if _which in ("all", "postnorm"):
     ext_modules.append(_ext("inference_gateway_amd.ops._postnorm",
                             postnorm_sources))
+if _which in ("all", "streams"):
+    ext_modules.append(_ext("inference_gateway_amd.ops._streams",
+                            streams_sources))
 
 setup(
     name="inference_gateway_amd_kernels",
