@@ -87,8 +87,9 @@ def parse_args():
     ap.add_argument("--arch", type=str, default="fedatar",
                     help="design for --arch-compare: fedatar or mekevik "
                          "(each beside Mixtral), feditar (beside "
-                         "Fedatar), bozolorn (beside Feditar) or "
-                         "bivatar (beside Fedatar)")
+                         "Fedatar), bozolorn (beside Feditar), "
+                         "bivatar (beside Fedatar) or defosun (beside "
+                         "Bozolorn)")
     ap.add_argument("--arch-size", type=str, default="2k",
                     help="layer shape for --arch-compare (2k | 4k)")
     ap.add_argument("--num-gpu-blocks", type=int, default=0,
@@ -523,6 +524,8 @@ def main() -> None:
             import bench_bozolorn as bench_hybrid
         elif args.arch == "bivatar":
             import bench_bivatar as bench_hybrid
+        elif args.arch == "defosun":
+            import bench_defosun as bench_hybrid
         else:
             import bench_hybrid
 

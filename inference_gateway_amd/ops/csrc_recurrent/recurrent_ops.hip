@@ -781,6 +781,63 @@ __global__ __launch_bounds__(256) void head_norm_gate_kernel(
   }
 }
 
+// wide groups (a norm over all heads together): a workgroup per (row,
+// group) pair, NV runs of four channels per thread in registers
+template <typename T, int NV>
+__global__ __launch_bounds__(256) void head_norm_gate_row_kernel(
+    T* __restrict__ out, const float* __restrict__ o,
+    const T* __restrict__ gate, int64_t gate_stride,
+    const float* __restrict__ w, const float* __restrict__ den,
+    const float* __restrict__ floor_, int H, int P, int group, float eps,
+    int gate_silu, int gate_first, int64_t npairs) {
+  __shared__ float red[8];
+  const int C = H * P;
+  const int ng = C / group;
+  const int t = blockIdx.x / ng, c0 = (blockIdx.x - t * ng) * group;
+  float val[NV][4], gz[NV][4];
+  float sq = 0.0f;
+#pragma unroll
+  for (int v = 0; v < NV; ++v) {
+    const int i = (v * 256 + threadIdx.x) * 4;
+    if (i < group)
+      hng_load<T, 4>(o + (int64_t)t * C + c0 + i,
+                     gate + (int64_t)t * gate_stride + c0 + i, val[v], gz[v]);
+    else
+#pragma unroll
+      for (int x = 0; x < 4; ++x) val[v][x] = gz[v][x] = 0.0f;
+  }
+#pragma unroll
+  for (int v = 0; v < NV; ++v) {
+    const int i = (v * 256 + threadIdx.x) * 4;
+    float scl = 1.0f;
+    if (den != nullptr && i < group) {
+      const int64_t h = (int64_t)t * H + (c0 + i) / P;   // P % 4 == 0
+      scl = 1.0f / (fmaxf(fabsf(den[h]), floor_ ? floor_[h] : 0.0f) + 1e-6f);
+    }
+#pragma unroll
+    for (int x = 0; x < 4; ++x) {
+      gz[v][x] = gate_value<T>(gz[v][x], gate_silu);
+      val[v][x] *= gate_first ? scl * gz[v][x] : scl;
+      sq += val[v][x] * val[v][x];
+    }
+  }
+  sq = block_reduce_sum<256>(sq, red);
+  const float rstd = 1.0f / sqrtf(sq / (float)group + eps);
+#pragma unroll
+  for (int v = 0; v < NV; ++v) {
+    const int i = (v * 256 + threadIdx.x) * 4;
+    if (i >= group) continue;
+    const float4 ww = *(const float4*)(w + c0 + i);
+    float r[4] = {val[v][0] * rstd * ww.x, val[v][1] * rstd * ww.y,
+                  val[v][2] * rstd * ww.z, val[v][3] * rstd * ww.w};
+    if (!gate_first)
+#pragma unroll
+      for (int x = 0; x < 4; ++x) r[x] *= gz[v][x];
+    Val4<T>::st(out + (int64_t)t * C + c0 + i,
+                make_float4(r[0], r[1], r[2], r[3]));
+  }
+}
+
 // any group size: one (row, group) pair per wave at a time, two passes
 template <typename T>
 __global__ __launch_bounds__(256) void head_norm_gate_wide_kernel(
@@ -873,12 +930,18 @@ void head_norm_gate(torch::Tensor out, torch::Tensor o, torch::Tensor gate,
   hipLaunchKernelGGL((head_norm_gate_kernel<act_t, VPL, VW>),                 \
                      dim3((npairs + 4 * HNG_PAIRS - 1) / (4 * HNG_PAIRS)),    \
                      dim3(256), 0, stream, HNG_ARGS)
+#define LAUNCH_HNG_ROW(NV)                                                    \
+  hipLaunchKernelGGL((head_norm_gate_row_kernel<act_t, NV>),                  \
+                     dim3((unsigned)npairs), dim3(256), 0, stream, HNG_ARGS)
   IGW_DISPATCH_ACT(out, {
     if (vec4 && group <= 64) LAUNCH_HNG(1, 1);
     else if (vec4 && group <= 128) LAUNCH_HNG(1, 2);
     else if (vec4 && group <= 256) LAUNCH_HNG(1, 4);
     else if (vec4 && group <= 512) LAUNCH_HNG(2, 4);
     else if (vec4 && group <= 1024) LAUNCH_HNG(4, 4);
+    else if (vec4 && group <= 2048) LAUNCH_HNG_ROW(2);
+    else if (vec4 && group <= 4096) LAUNCH_HNG_ROW(4);
+    else if (vec4 && group <= 8192) LAUNCH_HNG_ROW(8);
     else if (group <= 64) LAUNCH_HNG(1, 1);
     else if (group <= 128) LAUNCH_HNG(2, 1);
     else if (group <= 256) LAUNCH_HNG(4, 1);
@@ -887,6 +950,7 @@ void head_norm_gate(torch::Tensor out, torch::Tensor o, torch::Tensor gate,
                          dim3((npairs + 3) / 4), dim3(256), 0, stream,
                          HNG_ARGS);
   });
+#undef LAUNCH_HNG_ROW
 #undef LAUNCH_HNG
 #undef HNG_ARGS
   HIP_CHECK_KERNEL();

@@ -38,9 +38,11 @@ typedef __attribute__((ext_vector_type(8))) short fd_short8;
 typedef __attribute__((ext_vector_type(4))) short fd_short4;
 typedef __attribute__((ext_vector_type(4))) float fd_float4;
 
+// silu as the activation type holds it: both kernels see the same values
 template <typename T>
-DEVINLINE float silu_for(float z) {
-  return z * sigmoid_for<T>(z);
+DEVINLINE float silu_act(float z) {
+  const float y = z * sigmoid_for<T>(z);
+  return sizeof(T) == 2 ? bf16_to_f32(f32_to_bf16(y)) : y;
 }
 
 // ---------------------------------------------------------------------------
@@ -105,15 +107,15 @@ __global__ __launch_bounds__(256) void fixed_decay_step_kernel(
       const int t = i / N, n = i - t * N;
       const float x = Act<T>::ld(q + (c0 + t) * q_s0 + g * q_s1 + n);
       const float y = Act<T>::ld(k + (c0 + t) * k_s0 + g * k_s1 + n);
-      lq[i] = silu ? silu_for<T>(x) : x;
-      lk[i] = silu ? silu_for<T>(y) : y;
+      lq[i] = silu ? silu_act<T>(x) : x;
+      lk[i] = silu ? silu_act<T>(y) : y;
     }
     for (int i = tid; i < tc * FD_PT; i += 256) {
       const int t = i / FD_PT, c = i - t * FD_PT;
       float x = 0.0f;
       if (p0 + c < P) {
         x = Act<T>::ld(v + (c0 + t) * v_s0 + h * v_s1 + p0 + c);
-        if (silu) x = silu_for<T>(x);
+        if (silu) x = silu_act<T>(x);
       }
       lv[i] = x;
     }
@@ -295,7 +297,7 @@ __global__ __launch_bounds__(NW * 64) void fixed_decay_chunk_kernel(
     if (silu) {
 #pragma unroll
       for (int e = 0; e < 8; ++e)
-        x.v[e] = f32_to_bf16(silu_for<uint16_t>(bf16_to_f32(x.v[e])));
+        x.v[e] = f32_to_bf16(silu_act<uint16_t>(bf16_to_f32(x.v[e])));
     }
     return x;      // silu(0) = 0: padding stays zero
   };
