@@ -38,11 +38,33 @@ typedef __attribute__((ext_vector_type(8))) short fd_short8;
 typedef __attribute__((ext_vector_type(4))) short fd_short4;
 typedef __attribute__((ext_vector_type(4))) float fd_float4;
 
+// round to nearest even by the conversion instruction
+DEVINLINE uint16_t cvt_bf16(float x) {
+  return __builtin_bit_cast(uint16_t, (__bf16)x);
+}
+
+// two at a time: one instruction
+typedef __attribute__((ext_vector_type(2))) float fd_float2;
+typedef __attribute__((ext_vector_type(2))) __bf16 fd_bf2;
+typedef __attribute__((ext_vector_type(2))) unsigned short fd_ushort2;
+DEVINLINE fd_ushort2 cvt_bf16x2(float a, float b) {
+  return __builtin_bit_cast(
+      fd_ushort2, __builtin_convertvector(fd_float2{a, b}, fd_bf2));
+}
+
 // silu as the activation type holds it: both kernels see the same values
 template <typename T>
-DEVINLINE float silu_act(float z) {
-  const float y = z * sigmoid_for<T>(z);
-  return sizeof(T) == 2 ? bf16_to_f32(f32_to_bf16(y)) : y;
+DEVINLINE float silu_act(float z);
+template <>
+DEVINLINE float silu_act<float>(float z) {
+  return z * sigmoid_f32(z);
+}
+DEVINLINE float silu_fast(float z) {
+  return z * __builtin_amdgcn_rcpf(1.0f + __expf(-z));
+}
+template <>
+DEVINLINE float silu_act<uint16_t>(float z) {
+  return bf16_to_f32(cvt_bf16(silu_fast(z)));
 }
 
 // ---------------------------------------------------------------------------
@@ -179,10 +201,14 @@ constexpr int FD_C = 64;      // rows per chunk
 // 8 floats -> bf16 high parts and bf16 remainders
 DEVINLINE void split_pair(const float* x, fd_short8& hi, fd_short8& lo) {
 #pragma unroll
-  for (int e = 0; e < 8; ++e) {
-    const uint16_t b = f32_to_bf16(x[e]);
-    hi[e] = (short)b;
-    lo[e] = (short)f32_to_bf16(x[e] - bf16_to_f32(b));
+  for (int e = 0; e < 8; e += 2) {
+    const fd_ushort2 b = cvt_bf16x2(x[e], x[e + 1]);
+    const fd_ushort2 r = cvt_bf16x2(x[e] - bf16_to_f32(b[0]),
+                                    x[e + 1] - bf16_to_f32(b[1]));
+    hi[e] = (short)b[0];
+    hi[e + 1] = (short)b[1];
+    lo[e] = (short)r[0];
+    lo[e + 1] = (short)r[1];
   }
 }
 
@@ -190,17 +216,32 @@ DEVINLINE fd_float4 mfma_bf16(fd_short8 a, fd_short8 b, fd_float4 c) {
   return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0);
 }
 
-// two 8-byte LDS reads: entries {4g..4g+3} and {16+4g..16+4g+3} of a row
-DEVINLINE fd_short8 frag_perm(const uint16_t* row, int g) {
-  const fd_short4 a = *(const fd_short4*)(row + 4 * g);
-  const fd_short4 b = *(const fd_short4*)(row + 16 + 4 * g);
+// The transposed tiles hold FD_C rows of the chunk per key entry or value
+// column: 128 bytes, eight 16-byte pieces, piece c of row n stored at c ^
+// (n & 7) ^ (n >> 3 & 7).  Staging lanes write rows that are 8 apart,
+// operand reads touch 16 neighbouring rows: either way the lanes spread
+// over all banks.
+DEVINLINE int fd_swz(int n, int j) {
+  return n * FD_C + ((((j >> 3) ^ n ^ (n >> 3)) & 7) << 3) + (j & 7);
+}
+
+// Rows of q and k (NP entries): piece c at c ^ a row number that changes
+// every 256 bytes, for operand reads of 16 neighbouring rows.
+template <int NP>
+DEVINLINE int fd_row(int j, int n) {
+  return j * NP + ((((n >> 3) ^ (j / (128 / NP))) & (NP / 8 - 1)) << 3) +
+         (n & 7);
+}
+
+// entries {j0 + 4g ..} and {j0 + 16 + 4g ..} of four each
+DEVINLINE fd_short8 fd_join(fd_short4 a, fd_short4 b) {
   return fd_short8{a[0], a[1], a[2], a[3], b[0], b[1], b[2], b[3]};
 }
 
 // segment table, int32 [5][nseg]: first row, end row, sequence, first
 // segment of its sequence (0/1), last segment of its sequence (0/1)
 template <int NP, int NW, bool VEC, bool STATE_ONLY>
-__global__ __launch_bounds__(NW * 64) void fixed_decay_chunk_kernel(
+__global__ __launch_bounds__(NW * 64, NW / 2) void fixed_decay_chunk_kernel(
     float* __restrict__ out, const uint16_t* __restrict__ q, int64_t q_s0,
     int64_t q_s1, const uint16_t* __restrict__ k, int64_t k_s0, int64_t k_s1,
     const uint16_t* __restrict__ v, int64_t v_s0, int64_t v_s1,
@@ -210,22 +251,23 @@ __global__ __launch_bounds__(NW * 64) void fixed_decay_chunk_kernel(
     const int32_t* __restrict__ seq_slots, int H, int G, int N, int P,
     int silu) {
   constexpr int NTILE = NP / 16;
-  constexpr int RS = NP + 8;         // LDS row stride of q and k
-  constexpr int CS = FD_C + 8;       // ... of the transposed k and v
   constexpr int PT = NW * 16;
   constexpr int NQ = NP / 8 / NW > 0 ? NP / 8 / NW : 1;   // pieces per thread
+  constexpr int PG = NP / 8 < 8 ? NP / 8 : 8;   // neighbouring lanes' pieces
   __shared__ __attribute__((aligned(16))) uint16_t qs[STATE_ONLY ? 8
-                                                                 : FD_C * RS];
+                                                                 : FD_C * NP];
   __shared__ __attribute__((aligned(16))) uint16_t ks[STATE_ONLY ? 8
-                                                                 : FD_C * RS];
-  __shared__ __attribute__((aligned(16))) uint16_t kt[NP * CS];
-  __shared__ __attribute__((aligned(16))) uint16_t vt[PT * CS];
-  // weighted scores as operand fragments: [row tile][k step][hi|lo][lane]
+                                                                 : FD_C * NP];
+  __shared__ __attribute__((aligned(16))) uint16_t kt[NP * FD_C];
+  __shared__ __attribute__((aligned(16))) uint16_t vt[PT * FD_C];
+  // weighted scores as operand fragments [hi|lo][lane]: row tiles 0-3
+  // against rows 0-31, then row tiles 2-3 against rows 32-63
   __shared__ __attribute__((aligned(16)))
-  uint16_t af[STATE_ONLY ? 8 : 4 * 2 * 2 * 64 * 8];
+  uint16_t af[STATE_ONLY ? 8 : 6 * 2 * 64 * 8];
   __shared__ float pw[FD_C + 1];
-  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
-  const int l16 = lane & 15, g4 = lane >> 4;
+  int tid = threadIdx.x;
+  const int wave = tid >> 6, lane = tid & 63;
+  int l16 = lane & 15, g4 = lane >> 4;
   const int sg = blockIdx.z, h = blockIdx.y;
   const int row0 = segs[sg], row1 = segs[nseg + sg];
   const int seq = segs[2 * nseg + sg];
@@ -260,8 +302,8 @@ __global__ __launch_bounds__(NW * 64) void fixed_decay_chunk_kernel(
       }
   }
 
-  // staging: lane = row of the chunk, a thread takes NQ pieces of 8 key
-  // entries (piece = wave + NW * i) and two pieces of 8 value columns
+  // staging: PG (values: 8) neighbouring lanes take neighbouring pieces of
+  // 8 entries of one row, so a row's 128 bytes arrive in one request
   ushort8 qr[NQ], kr[NQ], vr[2];
   auto piece = [&](const uint16_t* base, int width, int c8, bool ok) {
     ushort8 x;
@@ -277,27 +319,42 @@ __global__ __launch_bounds__(NW * 64) void fixed_decay_chunk_kernel(
     }
     return x;
   };
+  auto k_place = [&](int i, int& j, int& c8) {
+    const int idx = tid + i * NW * 64;
+    j = (idx / PG) & (FD_C - 1);
+    c8 = (idx / (PG * FD_C) * PG + (idx & (PG - 1))) * 8;
+  };
+  auto v_place = [&](int i, int& j, int& c8) {
+    const int idx = tid + i * NW * 64;
+    j = (idx >> 3) & (FD_C - 1);
+    c8 = ((idx >> 9) * 8 + (idx & 7)) * 8;
+  };
   auto fetch = [&](int c0) {
-    const int64_t row = c0 + lane;
-    const bool ok = row < row1;
+    int j, c8;
 #pragma unroll
     for (int i = 0; i < NQ; ++i) {
-      const int c8 = (wave + NW * i) * 8;
-      const bool in = ok && c8 < NP;
+      k_place(i, j, c8);
+      const int64_t row = c0 + j;
+      const bool in = row < row1 && c8 < NP;
       kr[i] = piece(k + row * k_s0 + kh * k_s1, N, c8, in);
       if (!STATE_ONLY) qr[i] = piece(q + row * q_s0 + kh * q_s1, N, c8, in);
     }
 #pragma unroll
     for (int i = 0; i < 2; ++i) {
-      const int c8 = (wave + NW * i) * 8;
-      vr[i] = piece(v + row * v_s0 + h * v_s1 + p0, P - p0, c8, ok);
+      v_place(i, j, c8);
+      const int64_t row = c0 + j;
+      vr[i] = piece(v + row * v_s0 + h * v_s1 + p0, P - p0, c8, row < row1);
     }
   };
   auto act8 = [&](ushort8 x) {
     if (silu) {
 #pragma unroll
-      for (int e = 0; e < 8; ++e)
-        x.v[e] = f32_to_bf16(silu_act<uint16_t>(bf16_to_f32(x.v[e])));
+      for (int e = 0; e < 8; e += 2) {
+        const fd_ushort2 y = cvt_bf16x2(silu_fast(bf16_to_f32(x.v[e])),
+                                        silu_fast(bf16_to_f32(x.v[e + 1])));
+        x.v[e] = y[0];
+        x.v[e + 1] = y[1];
+      }
     }
     return x;      // silu(0) = 0: padding stays zero
   };
@@ -305,28 +362,32 @@ __global__ __launch_bounds__(NW * 64) void fixed_decay_chunk_kernel(
   fetch(row0);
   for (int c0 = row0; c0 < row1; c0 += FD_C) {
     const int L = min(FD_C, row1 - c0);
+    // LDS addresses are recomputed per chunk: kept across chunks they would
+    // cost half of the registers
+    if (NW == 8) asm volatile("" : "+v"(tid), "+v"(l16), "+v"(g4));
+    int j, c8;
 #pragma unroll
     for (int i = 0; i < NQ; ++i) {
-      const int c8 = (wave + NW * i) * 8;
+      k_place(i, j, c8);
       if (c8 < NP) {
         const ushort8 kk = act8(kr[i]);
 #pragma unroll
-        for (int e = 0; e < 8; ++e) kt[(c8 + e) * CS + lane] = kk.v[e];
+        for (int e = 0; e < 8; ++e) kt[fd_swz(c8 + e, j)] = kk.v[e];
         if (!STATE_ONLY) {
-          *(ushort8*)(ks + lane * RS + c8) = kk;
-          *(ushort8*)(qs + lane * RS + c8) = act8(qr[i]);
+          *(ushort8*)(ks + fd_row<NP>(j, c8)) = kk;
+          *(ushort8*)(qs + fd_row<NP>(j, c8)) = act8(qr[i]);
         }
       }
     }
 #pragma unroll
     for (int i = 0; i < 2; ++i) {
-      const int c8 = (wave + NW * i) * 8;
+      v_place(i, j, c8);
       const ushort8 vv = act8(vr[i]);
 #pragma unroll
-      for (int e = 0; e < 8; ++e) vt[(c8 + e) * CS + lane] = vv.v[e];
+      for (int e = 0; e < 8; ++e) vt[fd_swz(c8 + e, j)] = vv.v[e];
     }
     __syncthreads();
-    if (c0 + FD_C < row1) fetch(c0 + FD_C);
+    if (NW == 4 && c0 + FD_C < row1) fetch(c0 + FD_C);
 
     if (!STATE_ONLY) {
       // weighted scores of (16 rows i) x (32 rows j), transposed product
@@ -340,11 +401,11 @@ __global__ __launch_bounds__(NW * 64) void fixed_decay_chunk_kernel(
 #pragma unroll
         for (int ns = 0; ns < NP / 32; ++ns) {
           const fd_short8 b = *(const fd_short8*)(
-              qs + (it * 16 + l16) * RS + ns * 32 + g4 * 8);
+              qs + fd_row<NP>(it * 16 + l16, ns * 32 + g4 * 8));
 #pragma unroll
           for (int x = 0; x < 2; ++x) {
             const fd_short8 aa = *(const fd_short8*)(
-                ks + (kst * 32 + x * 16 + l16) * RS + ns * 32 + g4 * 8);
+                ks + fd_row<NP>(kst * 32 + x * 16 + l16, ns * 32 + g4 * 8));
             c[x] = mfma_bf16(aa, b, c[x]);
           }
         }
@@ -359,7 +420,7 @@ __global__ __launch_bounds__(NW * 64) void fixed_decay_chunk_kernel(
           }
         fd_short8 hi, lo;
         split_pair(w, hi, lo);
-        uint16_t* f = af + ((it * 2 + kst) * 2 * 64 + lane) * 8;
+        uint16_t* f = af + ((it + 2 * kst) * 2 * 64 + lane) * 8;
         *(fd_short8*)f = hi;
         *(fd_short8*)(f + 64 * 8) = lo;
       }
@@ -376,8 +437,10 @@ __global__ __launch_bounds__(NW * 64) void fixed_decay_chunk_kernel(
         split_pair(x, hi, lo);
 #pragma unroll
         for (int it = 0; it < 4; ++it) {
+          const int i = it * 16 + l16, n = ns * 32 + 4 * g4;
           const fd_short8 aa =
-              frag_perm(qs + (it * 16 + l16) * RS + ns * 32, g4);
+              fd_join(*(const fd_short4*)(qs + fd_row<NP>(i, n)),
+                      *(const fd_short4*)(qs + fd_row<NP>(i, n + 16)));
           acc[it] = mfma_bf16(aa, hi, acc[it]);
           acc[it] = mfma_bf16(aa, lo, acc[it]);
         }
@@ -391,13 +454,17 @@ __global__ __launch_bounds__(NW * 64) void fixed_decay_chunk_kernel(
       fd_short8 vb[2];
 #pragma unroll
       for (int kst = 0; kst < 2; ++kst)
-        vb[kst] = frag_perm(vt + (wave * 16 + l16) * CS + kst * 32, g4);
+        vb[kst] = fd_join(
+            *(const fd_short4*)(vt + fd_swz(wave * 16 + l16,
+                                            kst * 32 + 4 * g4)),
+            *(const fd_short4*)(vt + fd_swz(wave * 16 + l16,
+                                            kst * 32 + 16 + 4 * g4)));
 #pragma unroll
       for (int it = 0; it < 4; ++it)
 #pragma unroll
         for (int kst = 0; kst < 2; ++kst) {
           if (kst * 32 > it * 16 + 15) continue;
-          const uint16_t* f = af + ((it * 2 + kst) * 2 * 64 + lane) * 8;
+          const uint16_t* f = af + ((it + 2 * kst) * 2 * 64 + lane) * 8;
           acc[it] = mfma_bf16(*(const fd_short8*)f, vb[kst], acc[it]);
           acc[it] = mfma_bf16(*(const fd_short8*)(f + 64 * 8), vb[kst],
                               acc[it]);
@@ -412,6 +479,9 @@ __global__ __launch_bounds__(NW * 64) void fixed_decay_chunk_kernel(
           }
       }
     }
+    // two eight-wave workgroups share a compute unit and its registers: the
+    // next rows are requested when the read-out's registers are free
+    if (NW == 8 && c0 + FD_C < row1) fetch(c0 + FD_C);
     // memory after the chunk
     const float aL = pw[L];
 #pragma unroll
@@ -419,7 +489,7 @@ __global__ __launch_bounds__(NW * 64) void fixed_decay_chunk_kernel(
 #pragma unroll
     for (int js = 0; js < 2; ++js) {
       const fd_short8 raw = *(const fd_short8*)(
-          vt + (wave * 16 + l16) * CS + js * 32 + g4 * 8);
+          vt + fd_swz(wave * 16 + l16, js * 32 + g4 * 8));
       float x[8];
 #pragma unroll
       for (int e = 0; e < 8; ++e) {
@@ -431,7 +501,7 @@ __global__ __launch_bounds__(NW * 64) void fixed_decay_chunk_kernel(
 #pragma unroll
       for (int nt = 0; nt < NTILE; ++nt) {
         const fd_short8 aa = *(const fd_short8*)(
-            kt + (nt * 16 + l16) * CS + js * 32 + g4 * 8);
+            kt + fd_swz(nt * 16 + l16, js * 32 + g4 * 8));
         S[nt] = mfma_bf16(aa, hi, S[nt]);
         S[nt] = mfma_bf16(aa, lo, S[nt]);
       }
