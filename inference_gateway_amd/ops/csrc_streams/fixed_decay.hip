@@ -221,16 +221,20 @@ DEVINLINE fd_float4 mfma_bf16(fd_short8 a, fd_short8 b, fd_float4 c) {
 // (n & 7) ^ (n >> 3 & 7).  Staging lanes write rows that are 8 apart,
 // operand reads touch 16 neighbouring rows: either way the lanes spread
 // over all banks.
-DEVINLINE int fd_swz(int n, int j) {
-  return n * FD_C + ((((j >> 3) ^ n ^ (n >> 3)) & 7) << 3) + (j & 7);
+// Row n = 16 t + m (m < 16): t enters the piece by itself, so a lane's
+// address is one exclusive-or away from that of t = 0.
+DEVINLINE int fd_swz(int t, int m, int j) {
+  return t * 16 * FD_C + m * FD_C +
+         ((((j >> 3) ^ m ^ (m >> 3) ^ (2 * t)) & 7) << 3) + (j & 7);
 }
 
 // Rows of q and k (NP entries): piece c at c ^ a row number that changes
 // every 256 bytes, for operand reads of 16 neighbouring rows.
+// Row j = 16 t + m: the piece depends on m alone.
 template <int NP>
-DEVINLINE int fd_row(int j, int n) {
-  return j * NP + ((((n >> 3) ^ (j / (128 / NP))) & (NP / 8 - 1)) << 3) +
-         (n & 7);
+DEVINLINE int fd_row(int t, int m, int n) {
+  return t * 16 * NP + m * NP +
+         ((((n >> 3) ^ (m / (128 / NP))) & (NP / 8 - 1)) << 3) + (n & 7);
 }
 
 // entries {j0 + 4g ..} and {j0 + 16 + 4g ..} of four each
@@ -264,9 +268,12 @@ __global__ __launch_bounds__(NW * 64, NW / 2) void fixed_decay_chunk_kernel(
   // against rows 0-31, then row tiles 2-3 against rows 32-63
   __shared__ __attribute__((aligned(16)))
   uint16_t af[STATE_ONLY ? 8 : 6 * 2 * 64 * 8];
-  __shared__ float pw[FD_C + 1];
+  // powers of the decay behind as many zeros: pw[negative] = 0
+  __shared__ float pw_lds[2 * FD_C + 1];
+  float* pw = pw_lds + FD_C;
   int tid = threadIdx.x;
-  const int wave = tid >> 6, lane = tid & 63;
+  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const int lane = tid & 63;
   int l16 = lane & 15, g4 = lane >> 4;
   const int sg = blockIdx.z, h = blockIdx.y;
   const int row0 = segs[sg], row1 = segs[nseg + sg];
@@ -275,7 +282,10 @@ __global__ __launch_bounds__(NW * 64, NW / 2) void fixed_decay_chunk_kernel(
   const bool last = segs[4 * nseg + sg] != 0;
   const int kh = h / (H / G);
   const float a = decay[h];
-  if (tid <= FD_C) pw[tid] = tid == 0 ? 1.0f : powf(a, (float)tid);
+  for (int i = tid; i <= 2 * FD_C; i += NW * 64) {
+    const int e = i - FD_C;
+    pw_lds[i] = e < 0 ? 0.0f : e == 0 ? 1.0f : powf(a, (float)e);
+  }
   const int p0 = blockIdx.x * PT;
   const int pc = p0 + wave * 16 + l16;     // this lane's value column
   float* st = state + ((int64_t)seq_slots[seq] * H + h) * N * P;
@@ -329,22 +339,32 @@ __global__ __launch_bounds__(NW * 64, NW / 2) void fixed_decay_chunk_kernel(
     j = (idx >> 3) & (FD_C - 1);
     c8 = ((idx >> 9) * 8 + (idx & 7)) * 8;
   };
+  // one base per chunk for the whole workgroup, 32-bit offsets per lane
+  const int ks0 = (int)k_s0, qs0 = (int)q_s0, vs0 = (int)v_s0;
   auto fetch = [&](int c0) {
+    const uint16_t* kb = k + (int64_t)c0 * k_s0 + kh * k_s1;
+    const uint16_t* qb = q + (int64_t)c0 * q_s0 + kh * q_s1;
+    const uint16_t* vb = v + (int64_t)c0 * v_s0 + h * v_s1 + p0;
+    const int left = row1 - c0;
     int j, c8;
 #pragma unroll
     for (int i = 0; i < NQ; ++i) {
       k_place(i, j, c8);
-      const int64_t row = c0 + j;
-      const bool in = row < row1 && c8 < NP;
-      kr[i] = piece(k + row * k_s0 + kh * k_s1, N, c8, in);
-      if (!STATE_ONLY) qr[i] = piece(q + row * q_s0 + kh * q_s1, N, c8, in);
+      const bool in = j < left && c8 < NP;
+      kr[i] = piece(kb + j * ks0, N, c8, in);
+      if (!STATE_ONLY) qr[i] = piece(qb + j * qs0, N, c8, in);
     }
 #pragma unroll
     for (int i = 0; i < 2; ++i) {
       v_place(i, j, c8);
-      const int64_t row = c0 + j;
-      vr[i] = piece(v + row * v_s0 + h * v_s1 + p0, P - p0, c8, row < row1);
+      vr[i] = piece(vb + j * vs0, P - p0, c8, j < left);
     }
+  };
+  // eight entries of row j, transposed, from column c8 on (a multiple of 8)
+  auto put8 = [&](uint16_t* tile, int c8, int j, ushort8 x) {
+    const int at = c8 * FD_C + ((((j >> 3) ^ (c8 >> 3)) & 7) << 3) + (j & 7);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) tile[(at ^ (e << 3)) + e * FD_C] = x.v[e];
   };
   auto act8 = [&](ushort8 x) {
     if (silu) {
@@ -371,20 +391,18 @@ __global__ __launch_bounds__(NW * 64, NW / 2) void fixed_decay_chunk_kernel(
       k_place(i, j, c8);
       if (c8 < NP) {
         const ushort8 kk = act8(kr[i]);
-#pragma unroll
-        for (int e = 0; e < 8; ++e) kt[fd_swz(c8 + e, j)] = kk.v[e];
+        put8(kt, c8, j, kk);
         if (!STATE_ONLY) {
-          *(ushort8*)(ks + fd_row<NP>(j, c8)) = kk;
-          *(ushort8*)(qs + fd_row<NP>(j, c8)) = act8(qr[i]);
+          const int at = fd_row<NP>(j >> 4, j & 15, c8);
+          *(ushort8*)(ks + at) = kk;
+          *(ushort8*)(qs + at) = act8(qr[i]);
         }
       }
     }
 #pragma unroll
     for (int i = 0; i < 2; ++i) {
       v_place(i, j, c8);
-      const ushort8 vv = act8(vr[i]);
-#pragma unroll
-      for (int e = 0; e < 8; ++e) vt[fd_swz(c8 + e, j)] = vv.v[e];
+      put8(vt, c8, j, act8(vr[i]));
     }
     __syncthreads();
     if (NW == 4 && c0 + FD_C < row1) fetch(c0 + FD_C);
@@ -401,23 +419,22 @@ __global__ __launch_bounds__(NW * 64, NW / 2) void fixed_decay_chunk_kernel(
 #pragma unroll
         for (int ns = 0; ns < NP / 32; ++ns) {
           const fd_short8 b = *(const fd_short8*)(
-              qs + fd_row<NP>(it * 16 + l16, ns * 32 + g4 * 8));
+              qs + fd_row<NP>(it, l16, ns * 32 + g4 * 8));
 #pragma unroll
           for (int x = 0; x < 2; ++x) {
             const fd_short8 aa = *(const fd_short8*)(
-                ks + fd_row<NP>(kst * 32 + x * 16 + l16, ns * 32 + g4 * 8));
+                ks + fd_row<NP>(kst * 2 + x, l16, ns * 32 + g4 * 8));
             c[x] = mfma_bf16(aa, b, c[x]);
           }
         }
+        // a^{i-j}, zero for j > i
         float w[8];
-        const int i = it * 16 + l16;
+        const float* pij = pw + it * 16 + l16 - kst * 32 - g4 * 4;
 #pragma unroll
         for (int x = 0; x < 2; ++x)
 #pragma unroll
-          for (int r = 0; r < 4; ++r) {
-            const int j = kst * 32 + x * 16 + g4 * 4 + r;
-            w[x * 4 + r] = j <= i ? pw[i - j] * c[x][r] : 0.0f;
-          }
+          for (int r = 0; r < 4; ++r)
+            w[x * 4 + r] = pij[-(x * 16 + r)] * c[x][r];
         fd_short8 hi, lo;
         split_pair(w, hi, lo);
         uint16_t* f = af + ((it + 2 * kst) * 2 * 64 + lane) * 8;
@@ -437,10 +454,10 @@ __global__ __launch_bounds__(NW * 64, NW / 2) void fixed_decay_chunk_kernel(
         split_pair(x, hi, lo);
 #pragma unroll
         for (int it = 0; it < 4; ++it) {
-          const int i = it * 16 + l16, n = ns * 32 + 4 * g4;
+          const int n = ns * 32 + 4 * g4;
           const fd_short8 aa =
-              fd_join(*(const fd_short4*)(qs + fd_row<NP>(i, n)),
-                      *(const fd_short4*)(qs + fd_row<NP>(i, n + 16)));
+              fd_join(*(const fd_short4*)(qs + fd_row<NP>(it, l16, n)),
+                      *(const fd_short4*)(qs + fd_row<NP>(it, l16, n + 16)));
           acc[it] = mfma_bf16(aa, hi, acc[it]);
           acc[it] = mfma_bf16(aa, lo, acc[it]);
         }
@@ -455,9 +472,8 @@ __global__ __launch_bounds__(NW * 64, NW / 2) void fixed_decay_chunk_kernel(
 #pragma unroll
       for (int kst = 0; kst < 2; ++kst)
         vb[kst] = fd_join(
-            *(const fd_short4*)(vt + fd_swz(wave * 16 + l16,
-                                            kst * 32 + 4 * g4)),
-            *(const fd_short4*)(vt + fd_swz(wave * 16 + l16,
+            *(const fd_short4*)(vt + fd_swz(wave, l16, kst * 32 + 4 * g4)),
+            *(const fd_short4*)(vt + fd_swz(wave, l16,
                                             kst * 32 + 16 + 4 * g4)));
 #pragma unroll
       for (int it = 0; it < 4; ++it)
@@ -470,12 +486,15 @@ __global__ __launch_bounds__(NW * 64, NW / 2) void fixed_decay_chunk_kernel(
                               acc[it]);
         }
       if (pc < P) {
+        // uniform row base + one 32-bit lane offset
+        const int off = g4 * 4 * H * P + pc;
+        const int full = L == FD_C ? FD_C : L - g4 * 4;
 #pragma unroll
         for (int it = 0; it < 4; ++it)
 #pragma unroll
           for (int r = 0; r < 4; ++r) {
-            const int i = it * 16 + g4 * 4 + r;
-            if (i < L) out[((int64_t)(c0 + i) * H + h) * P + pc] = acc[it][r];
+            float* o = out + ((int64_t)(c0 + it * 16 + r) * H + h) * P;
+            if (it * 16 + r < full) o[off] = acc[it][r];
           }
       }
     }
@@ -489,19 +508,19 @@ __global__ __launch_bounds__(NW * 64, NW / 2) void fixed_decay_chunk_kernel(
 #pragma unroll
     for (int js = 0; js < 2; ++js) {
       const fd_short8 raw = *(const fd_short8*)(
-          vt + fd_swz(wave * 16 + l16, js * 32 + g4 * 8));
+          vt + fd_swz(wave, l16, js * 32 + g4 * 8));
+      // a^{L-1-j}; zero past the last row
       float x[8];
+      const float* pl = pw + L - 1 - js * 32 - g4 * 8;
 #pragma unroll
-      for (int e = 0; e < 8; ++e) {
-        const int j = js * 32 + g4 * 8 + e;
-        x[e] = j < L ? bf16_to_f32((uint16_t)raw[e]) * pw[L - 1 - j] : 0.0f;
-      }
+      for (int e = 0; e < 8; ++e)
+        x[e] = bf16_to_f32((uint16_t)raw[e]) * pl[-e];
       fd_short8 hi, lo;
       split_pair(x, hi, lo);
 #pragma unroll
       for (int nt = 0; nt < NTILE; ++nt) {
         const fd_short8 aa = *(const fd_short8*)(
-            kt + fd_swz(nt * 16 + l16, js * 32 + g4 * 8));
+            kt + fd_swz(nt, l16, js * 32 + g4 * 8));
         S[nt] = mfma_bf16(aa, hi, S[nt]);
         S[nt] = mfma_bf16(aa, lo, S[nt]);
       }
