@@ -513,6 +513,37 @@ def test_fixed_decay_segments_bf16(dims):
         assert np.abs(got - end).max() < 1e-3 * np.abs(end).max()
 
 
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("dims", [(3, 24, 1), (5, 7, 1), (18, 64, 1),
+                                  (12, 200, 2), (10, 300, 1), (16, 512, 1),
+                                  (3, 401, 1), (20, 512, 1)])
+def test_read_out_norm_over_many_channels(device, dims):
+    """One RMS norm over all heads together, or over half of them, times
+    the weight and the gate, with and without a normaliser per head."""
+    H, P, parts = dims
+    C = H * P
+    g = torch.Generator().manual_seed(C)
+    o = torch.randn(5, H, P, generator=g) * 3.0
+    gate = torch.randn(5, C + 8, generator=g)[:, :C]
+    w = torch.randn(C, generator=g)
+    den = torch.randn(5, H, generator=g)
+    dev = _dev(device)
+    for d, first, kind in ((None, False, ops.GATE_SIGMOID),
+                           (den, True, ops.GATE_SILU)):
+        a = f64(gate)
+        a = oracle.silu(a) if kind == ops.GATE_SILU else oracle.sigmoid(a)
+        y = f64(o)
+        if d is not None:
+            y = y / (np.abs(f64(d)) + 1e-6)[:, :, None]
+        y = y.reshape(5, C) * (a if first else 1.0)
+        y = oracle.rms_unit(y.reshape(5, parts, -1), 1e-5).reshape(5, C) \
+            * f64(w) * (1.0 if first else a)
+        got = ops.head_norm_gate(
+            o.to(dev), gate.to(dev), w.to(dev), 1e-5, C // parts, kind,
+            first, None if d is None else d.to(dev), None, torch.float32)
+        np.testing.assert_allclose(f64(got), y, atol=3e-5, rtol=1e-4)
+
+
 def test_decay_plan_covers_every_row_once():
     for rows in ((700,), (16, 15, 0, 64), (1, 1, 1), (5000, 3, 20),
                  (256, 256, 255)):
@@ -1031,3 +1062,26 @@ def test_trace_command(tmp_path):
     assert not (tmp_path / "o" / "1.f32").exists()
     close(g0, ra[[0, 4]], 2e-4)
     close(g2, np.stack([ra[8], rb[3]]), 2e-4)
+
+
+def test_bench_configurations_are_comparable():
+    """The speed comparison runs both models at equal width, head sizes
+    and routed experts, and its sizes run through the model."""
+    root = Path(__file__).resolve().parent.parent
+    sys.path.insert(0, str(root / "tools"))
+    try:
+        import bench_defosun as bd
+    finally:
+        sys.path.pop(0)
+    for sz in bd.SIZES.values():
+        dfo, boz = bd._configs(sz)
+        assert dfo.hidden_size == boz.hidden_size == sz["width"]
+        assert len(dfo.layer_runs) == boz.num_layers
+        a, b = dfo.layers[0].mixer, boz.layers[0].mixer.left
+        for k in ("heads", "kv_heads", "dim", "vdim"):
+            assert getattr(a, k) == getattr(b, k)
+        d, m = dfo.layers[1].mixer, boz.layers[0].mixer.right
+        assert (d.heads, d.dim, d.vdim) == (m.heads, m.dim, m.vdim)
+        for x, y in zip(dfo.layers, boz.layers):
+            for k in ("experts", "top", "expert_ff", "limit"):
+                assert getattr(x.mlp, k) == getattr(y.mlp, k)
