@@ -230,8 +230,8 @@ class LocalProvider:
         if local_cfg.model == "hf":
             # architecture straight from the checkpoint's config.json
             # (HuggingFace Llama-family layouts, or the per-layer Fedatar,
-            # Mekevik, Feditar, Bozolorn and Bivatar designs, which name
-            # themselves in config.json)
+            # Mekevik, Feditar, Bozolorn, Bivatar and Defosun designs, which
+            # name themselves in config.json)
             from ..engine.models.registry import model_config_from_dir
 
             preset = model_config_from_dir(weights)
